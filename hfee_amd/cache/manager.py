@@ -8,8 +8,8 @@ cache group, a block table (page ids by position // page_size) and one state slo
 
 Groups: layers whose caches have the same needs share a group and a page id
 addresses the same place in each of the group's layers.  A "full" group keeps every
-key; a "window" group keeps the last `window` keys, and pages that the window has
-passed go back to the pool at commit time.  A group with `every` = P > 1 grows by one
+key; a "window" group keeps the last `window` keys (and, with `keep_first`, the first ones
+of the sequence), and pages that the window has passed go back to the pool at commit time.  A group with `every` = P > 1 grows by one
 entry every P tokens (a pooled block of P tokens, say): a request of n tokens holds
 ceil(n / P) entries of it, in ceil(ceil(n / P) / page_size) pages.  Pages come back when a request is
 released and are handed out again at once (last freed, first reused).
@@ -56,12 +56,15 @@ class CacheGroupSpec:
     window: int = 0           # keys kept per token for kind == "window"
     layout: str = ""
     every: int = 1            # tokens an entry: the group grows by one entry every `every` tokens
+    keep_first: int = 0       # a window group's first tokens that are kept beside the window
 
     def __post_init__(self):
         if self.kind not in ("full", "window"):
             raise CacheError(f"unknown cache group kind {self.kind!r}")
         if self.kind == "window" and self.window <= 0:
             raise CacheError("a window group needs a positive window")
+        if int(self.keep_first) < 0 or (self.keep_first and self.kind != "window"):
+            raise CacheError("only a window group keeps its first tokens beside the window")
         if int(self.every) < 1 or (self.every > 1 and self.kind != "full"):
             raise CacheError("a group grows by one entry every `every` >= 1 tokens, and only a full group by fewer than one a token")
         if not self.token_shape or any(int(n) < 1 for n in self.token_shape):
@@ -331,7 +334,8 @@ class CacheManager:
             first_needed = max(0, rc.length - spec.window + 1)
             dead_until = first_needed // self.page_size        # blocks < dead_until are never read again
             table = rc.tables[g]
-            for b in range(rc.first_live_block[g], min(dead_until, len(table))):
+            kept = self._blocks_for(spec.keep_first, g)        # the sequence's first blocks stay
+            for b in range(max(rc.first_live_block[g], kept), min(dead_until, len(table))):
                 if table[b] >= 0:
                     self.pools[g].give_back(table[b], request_id)
                     table[b] = -1

@@ -76,12 +76,14 @@ class CacheNeed:
     `every` tokens (entry b belongs to the tokens b * every .. b * every + every - 1: a pooled block, a
     summary), and a request of n tokens holds ceil(n / every) entries of it.  A part that needs two kinds
     of growing memory answers `cache_spec()` with a tuple of needs; the first is the cache layer that the
-    schedule names, need k > 0 lives under the cache layer (that layer, k)."""
+    schedule names, need k > 0 lives under the cache layer (that layer, k).  `keep_first`: tokens from the
+    sequence's start that a "window" keeps beside its last ones."""
     kind: str                 # "full": every token is kept; "window": the last `window` tokens
     token_shape: tuple
     window: int = 0
     layout: str = ""
     every: int = 1
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)

@@ -48,31 +48,42 @@ inline int make_kv_layout(KvLayout* out, int kv_heads, int dk, int dv, int page_
   return 0;
 }
 
-// What a query at position p sees: the keys first_key(p) .. p, and the pooled blocks 0 .. pooled_blocks(p) - 1
+// What a query at position p sees: the keys first_key(p) .. p (behind a window the last `window` positions, within
+// chunks those of its own chunk, floor(p / chunk), counted from position 0), of the first `keep_first` positions
+// also those before first_key(p), and the pooled blocks 0 .. pooled_blocks(p) - 1
 // (block b holds the positions b * pool .. b * pool + pool - 1 and is seen once all of them have left the
 // window: b * pool + pool - 1 <= p - window).  The pooled blocks are a cache layer of their own, of the same
 // sizes and the same arrangement a page as the tokens', with block tables of its own: block b is its entry b.
 struct KeySight {
   int window;               // 0: every earlier position
+  int chunk;                // 0: none
+  int keep_first;           // the first tokens of a sequence that every later query sees
   int pool;                 // 0: no pooled blocks
   float softcap;            // 0: scores as they are
   const void* pooled;       // the pooled blocks' cache layer
   const int* pool_tables;   // its block tables, a row a segment as the tokens' have
   int pool_bt_stride;
 
-  __host__ __device__ __forceinline__ int first_key(int p) const { return window > 0 && p - window + 1 > 0 ? p - window + 1 : 0; }
+  __host__ __device__ __forceinline__ int first_key(int p) const {
+    const int behind = window > 0 && p - window + 1 > 0 ? p - window + 1 : 0;
+    const int own = chunk > 0 ? p - p % chunk : 0;
+    return behind > own ? behind : own;
+  }
   __host__ __device__ __forceinline__ int pooled_blocks(int p) const {
     return pool > 0 && window > 0 && p - window + 1 >= pool ? (p - window + 1) / pool : 0;
   }
   __device__ __forceinline__ float capped(float s) const { return softcap > 0.f ? softcap * tanhf(s / softcap) : s; }
 };
 
-inline int make_key_sight(KeySight* out, int window, int pool, float softcap, const void* pooled, const int* pool_tables,
-                          int pool_bt_stride) {
-  if (window < 0 || pool < 0 || !(softcap >= 0.f)) return fail("bad window %d, pool %d or softcap %f", window, pool, (double)softcap);
+inline int make_key_sight(KeySight* out, int window, int chunk, int keep_first, int pool, float softcap, const void* pooled,
+                          const int* pool_tables, int pool_bt_stride) {
+  if (window < 0 || chunk < 0 || keep_first < 0 || pool < 0 || !(softcap >= 0.f))
+    return fail("bad window %d, chunk %d, kept first keys %d, pool %d or softcap %f", window, chunk, keep_first, pool, (double)softcap);
   if (pool > 0 && window > 0 && (pooled == nullptr || pool_tables == nullptr))
     return fail("pooled blocks need their cache layer and its block tables");
   out->window = window;
+  out->chunk = chunk;
+  out->keep_first = keep_first;
   out->pool = window > 0 ? pool : 0;
   out->softcap = softcap;
   out->pooled = pooled;

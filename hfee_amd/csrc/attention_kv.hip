@@ -22,6 +22,9 @@
 // square over each head and multiplied by a weight shared by the heads, q also by a temperature that
 // grows with the logarithm of the position in steps of `every` tokens:
 // 1 + coef * ln(floor((p + 1) / every) + 1).
+//
+// qkv_write is the way with everything that may stand between a projection and its rotation: biases on q, k
+// and v, and the root mean square taken out of q and k, over each head or over all heads of a token at once.
 #include "attention_kv.h"
 
 using namespace hfee;
@@ -186,6 +189,88 @@ __global__ __launch_bounds__(256) void rotate_norm_write_kernel(
     cache[lay.value_offset(page, g, slot, d)] = finite_for_cache<T>(from_float<T>(p[d] * inv));
 }
 
+// ---------------------------------------------------------------- biases, norms, rotation, cache write
+// q (to q_out), k and v (into the token's slot) from their projections: x + bias (each optional, float32), then for q
+// and k with NORM 1 divided by the root mean square over the head and multiplied by a weight [dk] that the heads
+// share, with NORM 2 by the root mean square over all heads of the token and a weight [heads * dk]; then the first
+// 2 * half dims of a head are rotated (pairs (i, i + half), tables [positions][half]).  All in float32, one rounding
+// at the end.  Workgroup (token, part): the first `q_parts` parts deal a token's query heads among them, the
+// next `k_parts` its key heads, the rest its value heads; a wave takes a head at a time.  With NORM 2 every part
+// sums over the whole row itself, in one fixed order (q_out is therefore not q).
+template <typename T, int NORM>
+__global__ __launch_bounds__(256) void qkv_write_kernel(
+    T* __restrict__ q_out, int64_t ldqo, const T* __restrict__ q, int64_t ldq, int num_heads, const T* __restrict__ k,
+    int64_t ldk, const T* __restrict__ v, int64_t ldv, const float* __restrict__ q_bias, const float* __restrict__ k_bias,
+    const float* __restrict__ v_bias, const float* __restrict__ q_weight, const float* __restrict__ k_weight, float eps,
+    const float* __restrict__ cos_t, const float* __restrict__ sin_t, int half, const int* __restrict__ positions,
+    const int* __restrict__ token_segment, const int* __restrict__ block_tables, int bt_stride, T* __restrict__ cache,
+    KvLayout lay, int q_parts, int k_parts) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
+  const int pos = positions[t], dk = lay.dk;
+  const float* c = cos_t + (int64_t)pos * half;
+  const float* s = sin_t + (int64_t)pos * half;
+  const int part = blockIdx.y;
+  int page = 0, slot = 0;
+  if (part >= q_parts) {
+    page = block_tables[(int64_t)token_segment[t] * bt_stride + (pos >> lay.page_shift)];
+    slot = pos & (lay.page_size - 1);
+  }
+  if (part >= q_parts + k_parts) {                      // values
+    const int v_parts = gridDim.y - q_parts - k_parts;
+    const T* row = v + (int64_t)t * ldv;
+    for (int e = (part - q_parts - k_parts) * blockDim.x + threadIdx.x; e < lay.kv_heads * lay.dv; e += v_parts * blockDim.x) {
+      const int g = e / lay.dv, d = e - g * lay.dv;
+      const float x = to_float<T>(row[e]) + (v_bias != nullptr ? v_bias[e] : 0.f);
+      cache[lay.value_offset(page, g, slot, d)] = finite_for_cache<T>(from_float<T>(x));
+    }
+    return;
+  }
+  const bool is_q = part < q_parts;
+  const T* row = is_q ? q + (int64_t)t * ldq : k + (int64_t)t * ldk;
+  const float* bias = is_q ? q_bias : k_bias;
+  const float* weight = is_q ? q_weight : k_weight;
+  const int heads = is_q ? num_heads : lay.kv_heads, parts = is_q ? q_parts : k_parts;
+  float inv = 1.0f;
+  if constexpr (NORM == 2) {
+    float ss = 0.f;
+    for (int e = threadIdx.x; e < heads * dk; e += blockDim.x) {
+      const float x = to_float<T>(row[e]) + (bias != nullptr ? bias[e] : 0.f);
+      ss = fmaf(x, x, ss);
+    }
+    inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)(heads * dk) + eps);
+  }
+  for (int h = (is_q ? part : part - q_parts) * waves + wave; h < heads; h += parts * waves) {
+    const T* p = row + (int64_t)h * dk;
+    const float* b = bias != nullptr ? bias + (int64_t)h * dk : nullptr;
+    const float* w = weight != nullptr ? weight + (NORM == 2 ? (int64_t)h * dk : 0) : nullptr;
+    if constexpr (NORM == 1) {
+      float ss = 0.f;
+      for (int d = lane; d < dk; d += 64) {
+        const float x = to_float<T>(p[d]) + (b != nullptr ? b[d] : 0.f);
+        ss = fmaf(x, x, ss);
+      }
+      inv = 1.0f / sqrtf(wave_sum(ss) / (float)dk + eps);
+    }
+    auto value = [&](int d) {
+      const float x = (to_float<T>(p[d]) + (b != nullptr ? b[d] : 0.f)) * inv;
+      return w != nullptr ? x * w[d] : x;
+    };
+    auto turned = [&](int d) {
+      if (d < half) return value(d) * c[d] - value(d + half) * s[d];
+      if (d < 2 * half) return value(d) * c[d - half] + value(d - half) * s[d - half];
+      return value(d);
+    };
+    if (is_q) {
+      T* o = q_out + (int64_t)t * ldqo + (int64_t)h * dk;
+      for (int d = lane; d < dk; d += 64) o[d] = from_float<T>(turned(d));
+    } else {
+      T* o = cache + lay.key_offset(page, h, slot, 0);
+      for (int d = lane; d < dk; d += 64) o[d] = finite_for_cache<T>(from_float<T>(turned(d)));
+    }
+  }
+}
+
 // ---------------------------------------------------------------- pooled blocks
 // One wave a (token, key/value head, 64 of the key's and value's dims): a token at the last position of a block of `pool` positions
 // (position % pool == pool - 1) leaves the block's key and value in the pooled blocks' cache layer under
@@ -236,7 +321,8 @@ __global__ __launch_bounds__(256) void kv_pool_write_kernel(
 constexpr int kMaxDvPerLane = 16;     // value sizes up to 1,024
 
 // What a query sees besides the keys up to its own position (`KeySight`): with a window it sees the last
-// `window` positions, itself included; with pooled blocks it also sees, for every block of `pool`
+// `window` positions, itself included; within chunks the positions of its own chunk; the first `keep_first`
+// tokens of its sequence also from behind either; with pooled blocks it also sees, for every block of `pool`
 // positions that lies wholly before the window, one key and one value (the block's means, kept in the
 // pooled section of the cache under the block's number); a score may be capped as
 // cap * tanh(score / cap) before it is weighed.  Tokens and blocks share one softmax.
@@ -255,7 +341,7 @@ __global__ __launch_bounds__(64) void attention_kv_plain_kernel(
   const int kvh = h / (num_heads / lay.kv_heads);
   const int pos = positions[t];
   const int* bt = block_tables + (int64_t)token_segment[t] * bt_stride;
-  const int first = sight.first_key(pos), blocks = sight.pooled_blocks(pos);
+  const int first = sight.first_key(pos), blocks = sight.pooled_blocks(pos), kept = min(sight.keep_first, first);
   const T* pooled = static_cast<const T*>(sight.pooled);
   const int* pbt = sight.pool_tables + (int64_t)token_segment[t] * sight.pool_bt_stride;
 
@@ -273,6 +359,8 @@ __global__ __launch_bounds__(64) void attention_kv_plain_kernel(
   if (weighting == 0) {
     for (int base = 0; base < blocks; base += 64)
       if (base + lane < blocks) m = fmaxf(m, score(pooled, pbt, base + lane));
+    for (int base = 0; base < kept; base += 64)
+      if (base + lane < kept) m = fmaxf(m, score(cache, bt, base + lane));
     for (int base = first & ~63; base <= pos; base += 64) {
       const int j = base + lane;
       if (j >= first && j <= pos) m = fmaxf(m, score(cache, bt, j));
@@ -313,6 +401,7 @@ __global__ __launch_bounds__(64) void attention_kv_plain_kernel(
     }
   };
   if (blocks > 0) walk(pooled, pbt, 0, blocks - 1);
+  if (kept > 0) walk(cache, bt, 0, kept - 1);
   walk(cache, bt, first, pos);
   lsum = wave_sum(lsum);
   if (has_sink) lsum += expf(sink - m);
@@ -492,6 +581,53 @@ HFEE_API int hfee_rotate_norm_write(void* q_out, int64_t ldqo, const float* q, i
   return 0;
 }
 
+// norm: 0 none, 1 over each head (weights float32 [dk]), 2 over all heads of a token (weights float32 [heads * dk]).
+HFEE_API int hfee_qkv_write(void* q_out, int64_t ldqo, const void* q, int64_t ldq, int num_heads, const void* k, int64_t ldk,
+                            const void* v, int64_t ldv, int dtype, const float* q_bias, const float* k_bias,
+                            const float* v_bias, int norm, const float* q_weight, const float* k_weight, float eps,
+                            const float* cos_t, const float* sin_t, int half, int table_positions, int max_position,
+                            const int* positions, const int* token_segment, const int* block_tables, int bt_stride,
+                            void* cache, int kv_heads, int dk, int dv, int page_size, int n, hipStream_t stream) {
+  HFEE_REQUIRE(n >= 0 && num_heads > 0 && q != nullptr && q_out != nullptr && q != q_out, "qkv_write: bad arguments");
+  if (n == 0) return 0;
+  HFEE_REQUIRE(norm >= 0 && norm <= 2 && eps >= 0.f, "qkv_write: the norm is none (0), a head's (1) or a token's (2)");
+  HFEE_REQUIRE(half >= 0 && 2 * half <= dk && (half == 0 || (cos_t != nullptr && sin_t != nullptr)),
+               "qkv_write: the rotated dims do not fit the heads, or their tables are missing");
+  HFEE_REQUIRE(half == 0 || max_position < table_positions,
+               "qkv_write: position %d is beyond the rotation tables of %d positions", max_position, table_positions);
+  KvLayout lay;
+  if (make_kv_layout(&lay, kv_heads, dk, dv, page_size)) return 1;
+  HFEE_REQUIRE(ldq >= (int64_t)num_heads * dk && ldqo >= (int64_t)num_heads * dk, "qkv_write: q rows too short");
+  if (k != nullptr) {
+    HFEE_REQUIRE(v != nullptr && cache != nullptr && token_segment != nullptr && block_tables != nullptr,
+                 "qkv_write: k, v, the cache and the block tables come together");
+    HFEE_REQUIRE(ldk >= (int64_t)kv_heads * dk && ldv >= (int64_t)kv_heads * dv, "qkv_write: k/v rows too short");
+  }
+  // a wave a head where a head needs nothing of the others (or the tokens are few), fewer parts where every part
+  // has to sum over the whole row
+  int q_parts = (num_heads + 3) / 4, k_parts = k != nullptr ? (kv_heads + 3) / 4 : 0;
+  int v_parts = k != nullptr ? (kv_heads * dv + 255) / 256 : 0;
+  if (n >= 256 && norm == 2) {
+    q_parts = (q_parts + 3) / 4;
+    k_parts = (k_parts + 3) / 4;
+  }
+  if (n >= 256) v_parts = (v_parts + 3) / 4;
+  HFEE_REQUIRE(q_parts + k_parts + v_parts <= 65535, "qkv_write: too many heads");
+#define LAUNCH(T, NORM)                                                                                              \
+  qkv_write_kernel<T, NORM><<<dim3(n, q_parts + k_parts + v_parts), 256, 0, stream>>>((T*)q_out, ldqo, (const T*)q, ldq,\
+      num_heads, (const T*)k, ldk, (const T*)v, ldv, q_bias, k_bias, v_bias, q_weight, k_weight, eps, cos_t, sin_t, half,\
+      positions, token_segment, block_tables, bt_stride, (T*)cache, lay, q_parts, k_parts)
+#define PICK(T)                                                                                                      \
+  if (norm == 0) LAUNCH(T, 0); else if (norm == 1) LAUNCH(T, 1); else LAUNCH(T, 2)
+  if (dtype == 0) { PICK(float); }
+  else if (dtype == 1) { PICK(bf16_t); }
+  else return fail("qkv_write: unknown dtype %d", dtype);
+#undef PICK
+#undef LAUNCH
+  HFEE_CHECK_LAUNCH("qkv_write");
+  return 0;
+}
+
 HFEE_API int hfee_kv_pool_write(const void* cache, void* pooled, int dtype, int pool, const int* positions,
                                 const int* token_segment, const int* block_tables, int bt_stride, const int* pool_tables,
                                 int pool_bt_stride, int kv_heads, int dk, int dv, int page_size, int n, hipStream_t stream) {
@@ -517,11 +653,11 @@ HFEE_API int hfee_attention_kv_plain(void* out, int64_t ld_out, const void* q, i
                                      int dtype, const int* positions, const int* token_segment,
                                      const int* block_tables, int bt_stride, int num_heads, int kv_heads, int dk,
                                      int dv, int page_size, float scale, const float* sinks, int weighting, int window,
-                                     int pool, float softcap, const void* pooled, const int* pool_tables, int pool_bt_stride,
+                                     int chunk, int keep_first, int pool, float softcap, const void* pooled, const int* pool_tables, int pool_bt_stride,
                                      const void* gate, int64_t ld_gate, int n, hipStream_t stream) {
   HFEE_REQUIRE(n >= 0, "attention_kv_plain: bad token count");
   KeySight sight;
-  if (make_key_sight(&sight, window, pool, softcap, pooled, pool_tables, pool_bt_stride)) return 1;
+  if (make_key_sight(&sight, window, chunk, keep_first, pool, softcap, pooled, pool_tables, pool_bt_stride)) return 1;
   HFEE_REQUIRE(gate == nullptr || ld_gate >= num_heads, "attention_kv_plain: the gates' rows are too short");
   HFEE_REQUIRE(weighting == 0 || weighting == 1, "attention_kv_plain: the weights are a softmax's (0) or sigmoids (1)");
   if (n == 0) return 0;

@@ -16,12 +16,14 @@
 //      split over several waves, whose partial results a second kernel joins.
 // The sink joins the denominator once, at the very end.
 //
-// A query may see less than every earlier key (`KeySight`, attention_kv.h): the last `window` positions only,
+// A query may see less than every earlier key (`KeySight`, attention_kv.h): the last `window` positions only, or
+// those of its own chunk of positions, the first tokens of its sequence also from behind either,
 // and beside them one pooled key and value for every block of `pool` positions that lies wholly before the
 // window (a cache layer of their own with block tables of its own, under the block's number); a score may be capped as
 // cap * tanh(score / cap); a head's result may be multiplied by sigmoid of a gate.  The kernel then walks
-// the tiles of the pooled layer that any of its rows sees, and after them the token tiles from the one
-// that holds the first key of its first row's window; a key weighs where it lies within its row's bounds.
+// the tiles of the pooled layer that any of its rows sees, after them the tiles of the first tokens that every
+// query keeps in sight (those that lie before the next), and then the token tiles from the one that holds the
+// first key of its first row's window or chunk; a key weighs where it lies within its row's bounds.
 //
 // Compiled with -DHFEE_KV_WEIGHTS=1 there is no softmax: a visible key weighs sigmoid(score + b_h), b_h a
 // number a head (given where the softmax has its sinks), nothing is normalized over the keys, and the
@@ -80,9 +82,10 @@ struct ScoreScale {
   }
 };
 
-// `lo`, `hi`: the first and the last entry of the section that the lane's row sees.
+// `lo`, `hi`: the first and the last entry of the section that the lane's row sees; entries before `keep` are seen
+// also below `lo`.
 __device__ __forceinline__ void weigh_tile(f32x4 (&s)[2], float& reference, float& lsum, f32x4 (&acc)[VBLOCKS],
-                                           Operand& pop, int j0, int g, int lo, int hi, ScoreScale scaled, bool masked) {
+                                           Operand& pop, int j0, int g, int lo, int hi, int keep, ScoreScale scaled, bool masked) {
   if constexpr (SIGMOID) {      // `reference` is the head's number (in base 2), and stays
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb)
@@ -90,7 +93,7 @@ __device__ __forceinline__ void weigh_tile(f32x4 (&s)[2], float& reference, floa
       for (int i = 0; i < 4; ++i) {
         const float p = 1.0f / (1.0f + __builtin_amdgcn_exp2f(-(scaled(s[kb][i]) + reference)));
         const int j = j0 + kb * 16 + g * 4 + i;
-        s[kb][i] = masked && (j > hi || j < lo) ? 0.f : p;
+        s[kb][i] = masked && (j > hi || (j < lo && j >= keep)) ? 0.f : p;
       }
     pop.u = u32x4{pack_bf16(s[0][0], s[0][1]), pack_bf16(s[0][2], s[0][3]), pack_bf16(s[1][0], s[1][1]),
                   pack_bf16(s[1][2], s[1][3])};
@@ -103,7 +106,7 @@ __device__ __forceinline__ void weigh_tile(f32x4 (&s)[2], float& reference, floa
     for (int i = 0; i < 4; ++i) {
       float v = scaled(s[kb][i]);
       const int j = j0 + kb * 16 + g * 4 + i;
-      if (masked && (j > hi || j < lo)) v = -INFINITY;
+      if (masked && (j > hi || (j < lo && j >= keep))) v = -INFINITY;
       s[kb][i] = v;
       tmax = fmaxf(tmax, v);
     }
@@ -215,11 +218,18 @@ __global__ __launch_bounds__(256) void attention_kv_kernel(
     for (int vb = 0; vb < VBLOCKS; ++vb) acc[b][vb] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
 
-  // the tiles to walk: those of the pooled layer that any row sees, then the token tiles from the first
-  // key of the first row's window on (without a window or pooled blocks: the token tiles from the first)
+  // the tiles to walk: those of the pooled layer that any row sees, the kept first tokens' tiles before the
+  // next, then the token tiles from the first key of the first row's window or chunk on (without any of
+  // these: the token tiles from the first)
   const int pool_tiles = (sight.pooled_blocks(max_pos) + 31) >> 5;
   const int tile_lo = sight.first_key(pos0) >> 5;
-  const int ntiles = pool_tiles + (max_pos >> 5) + 1 - tile_lo;
+  const int kept_tiles = min((sight.keep_first + 31) >> 5, tile_lo);
+  const int ntiles = pool_tiles + kept_tiles + (max_pos >> 5) + 1 - tile_lo;
+  auto tile_of = [&](int walked) {
+    if (walked < pool_tiles) return walked;
+    const int t = walked - pool_tiles;
+    return t < kept_tiles ? t : tile_lo + t - kept_tiles;
+  };
   const int per_split = (ntiles + splits - 1) / splits;
   const int tile_begin = split * per_split, tile_end = min(ntiles, tile_begin + per_split);
   const int last_block = max_pos >> lay.page_shift;
@@ -232,7 +242,7 @@ __global__ __launch_bounds__(256) void attention_kv_kernel(
   // tile's two blocks of 16 keys; `values` gets where the lane's value columns of the two blocks begin
   auto load_keys = [&](int walked, Operand (&kop)[2][PIPE ? KSTEPS : 1], const bf16_t* (&values)[2]) {
     const bf16_t* section = walked < pool_tiles ? pooled : cache;
-    const int tile = walked < pool_tiles ? walked : tile_lo + walked - pool_tiles;
+    const int tile = tile_of(walked);
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) {
       const int jb = (tile << 5) + kb * 16;
@@ -250,7 +260,7 @@ __global__ __launch_bounds__(256) void attention_kv_kernel(
   // (without the second set, a key operand lives from its load to its products only)
   auto load_keys_of_block = [&](int walked, int kb, int st, const bf16_t*& values) {
     const bf16_t* section = walked < pool_tiles ? pooled : cache;
-    const int tile = walked < pool_tiles ? walked : tile_lo + walked - pool_tiles;
+    const int tile = tile_of(walked);
     const int jb = (tile << 5) + kb * 16;
     const int page = walked < pool_tiles ? pbt[min(jb >> lay.page_shift, last_pool_block)] : bt[min(jb >> lay.page_shift, last_block)];
     const int slot0 = jb & slot_mask;
@@ -268,7 +278,7 @@ __global__ __launch_bounds__(256) void attention_kv_kernel(
 
   for (int tile = tile_begin; tile < tile_end; ++tile) {
     const bool in_pool = tile < pool_tiles;
-    const int j0 = (in_pool ? tile : tile_lo + tile - pool_tiles) << 5;
+    const int j0 = tile_of(tile) << 5, keep = in_pool ? 0 : sight.keep_first;
     // which row blocks see any key of this tile (the same answer in every lane), and whether all their rows
     // see all of it: the entries that a row at position p sees are lo(p) .. hi(p), both growing with p
     bool live[RB], masked_tile[RB];
@@ -279,8 +289,8 @@ __global__ __launch_bounds__(256) void attention_kv_kernel(
       const int hi_first = in_pool ? sight.pooled_blocks(p_first) - 1 : p_first;
       const int hi_last = in_pool ? sight.pooled_blocks(p_last) - 1 : p_last;
       const int lo_first = in_pool ? 0 : sight.first_key(p_first), lo_last = in_pool ? 0 : sight.first_key(p_last);
-      live[b] = (MODE == 1 || b < blocks) && j0 <= hi_last && j0 + 31 >= lo_first;
-      masked_tile[b] = j0 + 31 > hi_first || j0 < lo_last;
+      live[b] = (MODE == 1 || b < blocks) && j0 <= hi_last && (j0 + 31 >= lo_first || j0 < keep);
+      masked_tile[b] = j0 + 31 > hi_first || (j0 < lo_last && j0 + 31 >= keep);
     }
     f32x4 s[RB][2];
     const bf16_t* vbase[2];
@@ -321,7 +331,7 @@ __global__ __launch_bounds__(256) void attention_kv_kernel(
       if (!live[b]) continue;
       const int lo = in_pool ? 0 : sight.first_key(pos[b]);
       const int hi = in_pool ? sight.pooled_blocks(pos[b]) - 1 : pos[b];
-      weigh_tile(s[b], m[b], lsum[b], acc[b], pop[b], j0, g, lo, hi, scaled, masked_tile[b]);
+      weigh_tile(s[b], m[b], lsum[b], acc[b], pop[b], j0, g, lo, hi, keep, scaled, masked_tile[b]);
     }
 #pragma unroll
     for (int vb = 0; vb < VBLOCKS; ++vb) {
@@ -442,11 +452,17 @@ __global__ __launch_bounds__(256) void attention_kv_shared_kernel(
     for (int vb = 0; vb < VBLOCKS; ++vb) acc[b][vb] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const int max_pos = pos0 + rows - 1;
-  // the tiles to walk: those of the pooled layer that any row sees, then the token tiles from the first key
-  // of the first row's window on
+  // the tiles to walk: those of the pooled layer that any row sees, the kept first tokens' tiles before the next,
+  // then the token tiles from the first key of the first row's window or chunk on
   const int pool_tiles = (sight.pooled_blocks(max_pos) + 31) >> 5;
   const int tile_lo = sight.first_key(pos0) >> 5;
-  const int ntiles = pool_tiles + (max_pos >> 5) + 1 - tile_lo;
+  const int kept_tiles = min((sight.keep_first + 31) >> 5, tile_lo);
+  const int ntiles = pool_tiles + kept_tiles + (max_pos >> 5) + 1 - tile_lo;
+  auto tile_of = [&](int walked) {
+    if (walked < pool_tiles) return walked;
+    const int t = walked - pool_tiles;
+    return t < kept_tiles ? t : tile_lo + t - kept_tiles;
+  };
   const int last_block = max_pos >> lay.page_shift;
   const int slot_mask = lay.page_size - 1;
   const bf16_t* const pooled = static_cast<const bf16_t*>(sight.pooled);
@@ -459,7 +475,7 @@ __global__ __launch_bounds__(256) void attention_kv_shared_kernel(
   u32x4 kst_a[kKeyLoads], vst_a[kValueLoads], kst_b[DEEP ? kKeyLoads : 1], vst_b[DEEP ? kValueLoads : 1];
   auto fetch = [&](int walked, u32x4* kst, u32x4* vst) {          // this thread's chunks of the tile, into registers
     const bf16_t* section = walked < pool_tiles ? pooled : cache;
-    const int tile = walked < pool_tiles ? walked : tile_lo + walked - pool_tiles;
+    const int tile = tile_of(walked);
     const bf16_t* keys[2];
     const bf16_t* values[2];
 #pragma unroll
@@ -501,7 +517,7 @@ __global__ __launch_bounds__(256) void attention_kv_shared_kernel(
   };
   auto multiply = [&](int walked, const bf16_t* st) {
     const bool in_pool = walked < pool_tiles;
-    const int j0 = (in_pool ? walked : tile_lo + walked - pool_tiles) << 5;
+    const int j0 = tile_of(walked) << 5, keep = in_pool ? 0 : sight.keep_first;
     // (the entries that a row at position p sees are lo(p) .. hi(p), both growing with p)
     bool live[RB], masked_tile[RB];
 #pragma unroll
@@ -510,8 +526,8 @@ __global__ __launch_bounds__(256) void attention_kv_shared_kernel(
       const int hi_first = in_pool ? sight.pooled_blocks(p_first) - 1 : p_first;
       const int hi_last = in_pool ? sight.pooled_blocks(p_last) - 1 : p_last;
       const int lo_first = in_pool ? 0 : sight.first_key(p_first), lo_last = in_pool ? 0 : sight.first_key(p_last);
-      live[b] = b < blocks && j0 <= hi_last && j0 + 31 >= lo_first;
-      masked_tile[b] = j0 + 31 > hi_first || j0 < lo_last;
+      live[b] = b < blocks && j0 <= hi_last && (j0 + 31 >= lo_first || j0 < keep);
+      masked_tile[b] = j0 + 31 > hi_first || (j0 < lo_last && j0 + 31 >= keep);
     }
     f32x4 s[RB][2];
 #pragma unroll
@@ -534,7 +550,7 @@ __global__ __launch_bounds__(256) void attention_kv_shared_kernel(
       if (!live[b]) continue;
       const int lo = in_pool ? 0 : sight.first_key(pos[b]);
       const int hi = in_pool ? sight.pooled_blocks(pos[b]) - 1 : pos[b];
-      weigh_tile(s[b], m[b], lsum[b], acc[b], pop[b], j0, g, lo, hi, scaled, masked_tile[b]);
+      weigh_tile(s[b], m[b], lsum[b], acc[b], pop[b], j0, g, lo, hi, keep, scaled, masked_tile[b]);
     }
 #pragma unroll
     for (int vb = 0; vb < VBLOCKS; ++vb) {
@@ -650,12 +666,13 @@ HFEE_API int hfee_attention_kv_bf16(void* out, int64_t ld_out, const void* q, in
                                     const int* items, int num_items, int mode, const int* block_tables,
                                     int bt_stride, int num_heads, int kv_heads, int page_size, float scale,
                                     const float* sinks, float* partial, int64_t partial_words, int splits,
-                                    int window, int pool, float softcap, const void* pooled, const int* pool_tables,
+                                    int window, int chunk, int keep_first, int pool, float softcap, const void* pooled,
+                                    const int* pool_tables,
                                     int pool_bt_stride, const void* gate,
                                     int64_t ld_gate, hipStream_t stream) {
   HFEE_REQUIRE(num_items >= 0, "attention_kv_bf16: bad item count");
   KeySight sight;
-  if (make_key_sight(&sight, window, pool, softcap, pooled, pool_tables, pool_bt_stride)) return 1;
+  if (make_key_sight(&sight, window, chunk, keep_first, pool, softcap, pooled, pool_tables, pool_bt_stride)) return 1;
   HFEE_REQUIRE(pooled == nullptr || (uintptr_t)pooled % 16 == 0, "attention_kv_bf16: the pooled layer must be aligned for vector access");
   HFEE_REQUIRE(gate == nullptr || ld_gate >= num_heads, "attention_kv_bf16: the gates' rows are too short");
   if (num_items == 0) return 0;

@@ -138,7 +138,26 @@ __device__ __forceinline__ void store4<bf16_t>(bf16_t* p, const float (&v)[4]) {
 // small: g/2 (1 + tanh y) = g / (1 + exp(-2y)), and the error function by its rational
 // approximation with exp(-x^2) (Abramowitz and Stegun 7.1.26, absolute error below 1.5e-7;
 // the kernels that use these round the result to bfloat16).
-enum { GATE_SILU = 0, GATE_GELU_TANH = 1, GATE_GELU = 2, GATE_RELU = 3, GATE_KINDS = 4 };
+// GATE_CLIPPED is not an activation of the gate alone: with the two numbers `limit` and `sharpness`,
+// g = min(gate, limit), u = clamp(up, -limit, limit), the product is g sigmoid(sharpness g) (u + 1).
+enum { GATE_SILU = 0, GATE_GELU_TANH = 1, GATE_GELU = 2, GATE_RELU = 3, GATE_CLIPPED = 4, GATE_KINDS = 5 };
+
+struct GateNumbers {
+  float limit, sharpness;      // of GATE_CLIPPED; the other activations have none
+};
+
+__device__ __forceinline__ float clipped_gate(float g, float u, GateNumbers k) {
+  g = fminf(g, k.limit);
+  u = fminf(fmaxf(u, -k.limit), k.limit);
+  return g * __frcp_rn(1.0f + __expf(-k.sharpness * g)) * (u + 1.0f);
+}
+
+// (to the last bit of the library's exponential, for the 32-bit path)
+__device__ __forceinline__ float clipped_gate_exact(float g, float u, GateNumbers k) {
+  g = fminf(g, k.limit);
+  u = fminf(fmaxf(u, -k.limit), k.limit);
+  return g / (1.0f + expf(-k.sharpness * g)) * (u + 1.0f);
+}
 
 template <int ACT>
 __device__ __forceinline__ float gate_other_as(float g) {

@@ -243,19 +243,24 @@ HFEE_API int hfee_rmsnorm(void* out, int out_dtype, const float* x, const void* 
 // ------------------------------------------------------------------ SiLU gate
 template <typename T>
 __global__ void swiglu_kernel(T* __restrict__ out, int64_t ld_out, const T* __restrict__ gate,
-                              const T* __restrict__ up, int64_t ld_in, int col_stride, int width, int act) {
+                              const T* __restrict__ up, int64_t ld_in, int col_stride, int width, int act,
+                              GateNumbers numbers) {
   const int row = blockIdx.y;
   const int j = blockIdx.x * blockDim.x + threadIdx.x;
   if (j >= width) return;
   const float g = to_float<T>(gate[(int64_t)row * ld_in + (int64_t)j * col_stride]);
   const float u = to_float<T>(up[(int64_t)row * ld_in + (int64_t)j * col_stride]);
-  out[(int64_t)row * ld_out + j] = from_float<T>((act == GATE_SILU ? g / (1.0f + expf(-g)) : gate_other_exact(g, act)) * u);
+  out[(int64_t)row * ld_out + j] = from_float<T>(act == GATE_CLIPPED ? clipped_gate_exact(g, u, numbers)
+                                                 : (act == GATE_SILU ? g / (1.0f + expf(-g)) : gate_other_exact(g, act)) * u);
 }
 
 // col_stride: distance between consecutive gate (and up) columns: 1 for two separate
-// blocks, 2 when gate and up alternate.  act: the gate's activation (GATE_SILU ...).
+// blocks, 2 when gate and up alternate.  act: the gate's activation (GATE_SILU ..., with its two numbers
+// where it has any).
 HFEE_API int hfee_swiglu(void* out, int64_t ld_out, const void* gate, const void* up, int64_t ld_in,
-                         int col_stride, int dtype, int n, int width, int act, hipStream_t stream) {
+                         int col_stride, int dtype, int n, int width, int act, float limit, float sharpness,
+                         hipStream_t stream) {
+  const GateNumbers numbers{limit, sharpness};
   HFEE_REQUIRE(act >= 0 && act < GATE_KINDS, "swiglu: unknown activation %d", act);
   HFEE_REQUIRE(n >= 0 && width > 0 && ld_out >= width && col_stride >= 1 &&
                ld_in >= (int64_t)(width - 1) * col_stride + 1, "swiglu: bad sizes");
@@ -268,11 +273,11 @@ HFEE_API int hfee_swiglu(void* out, int64_t ld_out, const void* gate, const void
     if (dtype == DT_F32)
       swiglu_kernel<float><<<grid, 256, 0, stream>>>((float*)out + row0 * ld_out, ld_out,
                                                      (const float*)gate + row0 * ld_in,
-                                                     (const float*)up + row0 * ld_in, ld_in, col_stride, width, act);
+                                                     (const float*)up + row0 * ld_in, ld_in, col_stride, width, act, numbers);
     else if (dtype == DT_BF16)
       swiglu_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)out + row0 * ld_out, ld_out,
                                                       (const bf16_t*)gate + row0 * ld_in,
-                                                      (const bf16_t*)up + row0 * ld_in, ld_in, col_stride, width, act);
+                                                      (const bf16_t*)up + row0 * ld_in, ld_in, col_stride, width, act, numbers);
     else
       return fail("swiglu: unknown dtype %d", dtype);
   }

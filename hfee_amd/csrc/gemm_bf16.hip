@@ -173,12 +173,20 @@ __device__ __forceinline__ float gated(float g) {
   else return gate_other_as<ACT>(g);
 }
 
+// The gate times what it gates.
+template <int ACT>
+__device__ __forceinline__ float gate_product(float g, float u, GateNumbers k) {
+  if constexpr (ACT == GATE_CLIPPED) return clipped_gate(g, u, k);
+  else return gated<ACT>(g) * u;
+}
+
 // Calls f(std::integral_constant<int, ACT>) for the activation of a gating product (MODE says whether it is one).
 template <int MODE, typename F>
 __device__ __forceinline__ void with_gate_activation(int act, F&& f) {
   if (MODE != OUT_SWIGLU || act == GATE_SILU) f(std::integral_constant<int, GATE_SILU>{});
   else if (act == GATE_GELU_TANH) f(std::integral_constant<int, GATE_GELU_TANH>{});
   else if (act == GATE_GELU) f(std::integral_constant<int, GATE_GELU>{});
+  else if (act == GATE_CLIPPED) f(std::integral_constant<int, GATE_CLIPPED>{});
   else f(std::integral_constant<int, GATE_RELU>{});
 }
 
@@ -200,7 +208,7 @@ struct TileOf {
 // bfloat16).  m: this lane's row of C (m_base + l % R).
 template <int MODE, int ACT = GATE_SILU, typename ACC>
 __device__ __forceinline__ void store_tile_t(void* C, int64_t ldc, int M, int N, int m, int n_base, int lane,
-                                             const ACC& t, bool vec) {
+                                             const ACC& t, bool vec, GateNumbers numbers = GateNumbers{0.f, 0.f}) {
   using T = TileOf<ACC>;
   if (m >= M) return;
 #pragma unroll
@@ -210,8 +218,8 @@ __device__ __forceinline__ void store_tile_t(void* C, int64_t ldc, int M, int N,
     float v[4] = {t[4 * q], t[4 * q + 1], t[4 * q + 2], t[4 * q + 3]};
     if (MODE == OUT_SWIGLU) {          // columns n, n+1 are gate, up of output column n / 2
       bf16_t* c = (bf16_t*)C + (int64_t)m * ldc + (n >> 1);
-      const bf16_t o0 = float_to_bf16(gated<ACT>(v[0]) * v[1]);
-      const bf16_t o1 = float_to_bf16(gated<ACT>(v[2]) * v[3]);
+      const bf16_t o0 = float_to_bf16(gate_product<ACT>(v[0], v[1], numbers));
+      const bf16_t o1 = float_to_bf16(gate_product<ACT>(v[2], v[3], numbers));
       if (vec && n + 3 < N) {
         *reinterpret_cast<uint32_t*>(c) = (uint32_t)o0 | ((uint32_t)o1 << 16);
       } else {
@@ -264,7 +272,8 @@ struct Stage {
 
 template <int MODE, int TM, int TN, int ACT = GATE_SILU, typename ACC>
 __device__ __forceinline__ void store_wave_staged(char* lds, void* C, int64_t ldc, int M, int m_first, int n_first,
-                                                  int lane, const ACC (&acc)[TM][TN]) {
+                                                  int lane, const ACC (&acc)[TM][TN],
+                                                  GateNumbers numbers = GateNumbers{0.f, 0.f}) {
   using T = TileOf<ACC>;
   constexpr int R = T::R;
   using S = Stage<MODE, TN, R>;
@@ -303,8 +312,8 @@ __device__ __forceinline__ void store_wave_staged(char* lds, void* C, int64_t ld
         const float v[4] = {t[4 * q], t[4 * q + 1], t[4 * q + 2], t[4 * q + 3]};
         const int col = j * R + T::STEP * q + 4 * h;          // this group's first column within the strip
         if constexpr (MODE == OUT_SWIGLU) {
-          const bf16_t o0 = float_to_bf16(gated<ACT>(v[0]) * v[1]);
-          const bf16_t o1 = float_to_bf16(gated<ACT>(v[2]) * v[3]);
+          const bf16_t o0 = float_to_bf16(gate_product<ACT>(v[0], v[1], numbers));
+          const bf16_t o1 = float_to_bf16(gate_product<ACT>(v[2], v[3], numbers));
           *reinterpret_cast<uint32_t*>(mine + (col / 2) * 2) = (uint32_t)o0 | ((uint32_t)o1 << 16);
         } else if constexpr (MODE == OUT_BF16) {
           u32x2 o;
@@ -559,7 +568,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_pipelined_kernel(void* __restri
 #pragma unroll
         for (int j = 0; j < TN; ++j)
           store_tile_t<MODE, decltype(act)::value>(C, ldc, M, N, m0 + wm * 32 * TM + i * 32 + lrow, n0 + wn * 32 * TN + j * 32,
-                                                   lane, acc[i][j], vec);
+                                                   lane, acc[i][j], vec, qkv.gate_numbers);
     });
   }
 }
@@ -1045,13 +1054,15 @@ __global__ __launch_bounds__(256) void gemm_bf16_direct_kernel(void* __restrict_
     with_gate_activation<MODE>(qkv.gate_act, [&](auto act) {
       constexpr int ACT = decltype(act)::value;
       if (whole_rows) {
-        store_wave_staged<MODE, TM16, TN16, ACT>(lds_bytes + wave * S::BYTES, C, ldc, M, m0 + wm * 32 * TM, n0 + wn * 32 * TN, lane, acc);
+        store_wave_staged<MODE, TM16, TN16, ACT>(lds_bytes + wave * S::BYTES, C, ldc, M, m0 + wm * 32 * TM, n0 + wn * 32 * TN, lane, acc,
+                                                  qkv.gate_numbers);
       } else {
 #pragma unroll
         for (int i = 0; i < TM16; ++i)
 #pragma unroll
           for (int j = 0; j < TN16; ++j)
-            store_tile_t<MODE, ACT>(C, ldc, M, N, m0 + wm * 32 * TM + i * 16 + lrow, n0 + wn * 32 * TN + j * 16, lane, acc[i][j], vec);
+            store_tile_t<MODE, ACT>(C, ldc, M, N, m0 + wm * 32 * TM + i * 16 + lrow, n0 + wn * 32 * TN + j * 16, lane, acc[i][j], vec,
+                                    qkv.gate_numbers);
       }
     });
   }
@@ -1239,13 +1250,15 @@ __global__ __launch_bounds__(256) void gemm_bf16_direct64_kernel(void* __restric
     with_gate_activation<MODE>(qkv.gate_act, [&](auto act) {
       constexpr int ACT = decltype(act)::value;
       if (whole_rows) {
-        store_wave_staged<MODE, TM16, TN16, ACT>(lds_bytes + wave * S::BYTES, C, ldc, M, m0 + wm * 32 * TM, n0 + wn * 32 * TN, lane, acc);
+        store_wave_staged<MODE, TM16, TN16, ACT>(lds_bytes + wave * S::BYTES, C, ldc, M, m0 + wm * 32 * TM, n0 + wn * 32 * TN, lane, acc,
+                                                  qkv.gate_numbers);
       } else {
 #pragma unroll
         for (int i = 0; i < TM16; ++i)
 #pragma unroll
           for (int j = 0; j < TN16; ++j)
-            store_tile_t<MODE, ACT>(C, ldc, M, N, m0 + wm * 32 * TM + i * 16 + lrow, n0 + wn * 32 * TN + j * 16, lane, acc[i][j], vec);
+            store_tile_t<MODE, ACT>(C, ldc, M, N, m0 + wm * 32 * TM + i * 16 + lrow, n0 + wn * 32 * TN + j * 16, lane, acc[i][j], vec,
+                                    qkv.gate_numbers);
       }
     });
   }
@@ -1515,14 +1528,15 @@ HFEE_API int hfee_gemm_bf16_scratch(int M, int N, int K) {
 // C = A W^T for bfloat16 A [M, K] and W [N, K].
 // out_mode: 0 bfloat16 store, 1 float32 store, 2 float32 accumulate, 3 gate (the
 // rows of W alternate gate/up; C is [M, N/2] bfloat16 = activation(gate) * up, the
-// activation being gate_act: GATE_SILU ...; aligned operands only).
+// activation being gate_act: GATE_SILU ..., with its two numbers where it has any; aligned operands only).
 // force_kernel: 0 choose by the sizes, 1 skinny, 2 tiled 128 x 128, 3 the simple tiled
 // kernel, 4 tiled 256 x 256, 5 tiled 256 x 128, 6 tiled 256 x 192, 7 tiled 128 x 128 and 8 tiled 128 x 192 loaded
 // straight into LDS (for tests of each kernel alone; 4 to 8 fall back to 2 where they do not apply).
 // scratch: null, or hfee_gemm_bf16_scratch(M, N, K) float32 words, 16-byte aligned.
 HFEE_API int hfee_gemm_bf16(void* C, int out_mode, int64_t ldc, const void* A, int64_t lda, const void* W,
                             int64_t ldw, int M, int N, int K, int force_kernel, float* scratch,
-                            int64_t scratch_floats, int gate_act, hipStream_t stream) {
+                            int64_t scratch_floats, int gate_act, float gate_limit, float gate_sharpness,
+                            hipStream_t stream) {
   Partial partial;
   partial.at = scratch;
   partial.floats = scratch != nullptr ? scratch_floats : 0;
@@ -1539,6 +1553,7 @@ HFEE_API int hfee_gemm_bf16(void* C, int out_mode, int64_t ldc, const void* A, i
     HFEE_REQUIRE(gate_act >= 0 && gate_act < GATE_KINDS, "gemm_bf16: unknown activation %d", gate_act);
     QkvArgs gate{};
     gate.gate_act = gate_act;
+    gate.gate_numbers = GateNumbers{gate_limit, gate_sharpness};
     if (launch_aligned<OUT_SWIGLU>(C, ldc, (const bf16_t*)A, lda, (const bf16_t*)W, ldw, M, N, K, force_kernel, stream, gate)) return 1;
     HFEE_CHECK_LAUNCH("gemm_bf16");
     return 0;
@@ -1593,7 +1608,7 @@ HFEE_API int hfee_gemm_bf16_add_norm(float* C, const void* A, int64_t lda, const
       return hfee_rmsnorm(normed, DT_BF16, C, norm_weight, norm_weight_is_f32 ? DT_F32 : DT_BF16, nullptr, eps, M, N, stream);
     }
   }
-  if (int rc = hfee_gemm_bf16(C, OUT_ADD_F32, N, A, lda, W, ldw, M, N, K, 0, scratch, scratch_floats, GATE_SILU, stream)) return rc;
+  if (int rc = hfee_gemm_bf16(C, OUT_ADD_F32, N, A, lda, W, ldw, M, N, K, 0, scratch, scratch_floats, GATE_SILU, 0.f, 0.f, stream)) return rc;
   return hfee_rmsnorm(normed, DT_BF16, C, norm_weight, norm_weight_is_f32 ? DT_F32 : DT_BF16, nullptr, eps, M, N, stream);
 }
 

@@ -7,12 +7,15 @@
 //   up:    act[t][j][f] = silu(W_gate[e][f] . h_t) * (W_up[e][f] . h_t),   e = the j-th expert of t
 //   down:  x[t][c] (+)= sum_j weight_tj (W_down[e_j][c] . act[t][j])
 //
+// With gate_act GATE_CLIPPED the experts' gate is the clipped one of common.h (two numbers, `limit` and `sharpness`).
+//
 // Experts without a gate (`form` 1, no W_gate): act[t][j][f] = relu(w_tj (W_up[e][f] . h_t))^2, where w_tj
 // (in_weights, or one) multiplies the expert's input: a product is linear, so the number meets the sum in
 // float32 before the activation instead of every element of h before it is rounded.
 //
-// router_topk: scores sigmoid(z) of router logits z (float32 [n, experts]); the `top` largest choose a
-// token's experts (the lower number of two equal ones), its pair weights are the chosen scores as they are.
+// router_topk: scores of router logits z (float32 [n, experts], plus a bias an expert where one is given); the
+// `top` largest choose a token's experts (the lower number of two equal ones), its pair weights are the chosen
+// scores: sigmoids, or the softmax over all experts, as they are, or the softmax over the chosen ones only.
 //
 // The experts' matrices are stacked [experts][rows][columns].  Two forms:
 //
@@ -81,7 +84,8 @@ __global__ __launch_bounds__(256) void moe_up_kernel(T* __restrict__ act, const 
                                                      const T* __restrict__ w_gate, const T* __restrict__ w_up,
                                                      const int* __restrict__ chosen, const int* __restrict__ table,
                                                      const int* __restrict__ token_ids, int top, int experts, int F,
-                                                     int width, const float* __restrict__ in_weights) {
+                                                     int width, const float* __restrict__ in_weights, int gate_act,
+                                                     GateNumbers numbers) {
   const int pair = blockIdx.x, t = pair / top, j = pair - t * top;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int e = expert_of(chosen, table, token_ids, t, j, top);
@@ -106,7 +110,9 @@ __global__ __launch_bounds__(256) void moe_up_kernel(T* __restrict__ act, const 
     two_dots<T>(g, u, hr, width, lane, wide, sg, su);
     sg = wave_sum(sg);
     su = wave_sum(su);
-    if (lane == 0) act[(int64_t)pair * F + f] = from_float<T>(sg / (1.0f + expf(-sg)) * su);
+    if (lane == 0)
+      act[(int64_t)pair * F + f] = from_float<T>(gate_act == GATE_CLIPPED ? clipped_gate_exact(sg, su, numbers)
+                                                                          : sg / (1.0f + expf(-sg)) * su);
   }
 }
 
@@ -198,7 +204,7 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(int* __restrict__ order
 // matrix) x 64 pairs as 2 x 2 tiles of `32x32x16`, the weights as the row operand, so that a lane ends with
 // four neighbouring rows of the matrix for one pair and stores them at once.  A sum runs over K in the same
 // order whichever pairs share the tile.
-//   KIND 0: act = silu(gate) * up      KIND 1: act = relu(weight * up)^2      KIND 2: out (+)= scale * down
+//   KIND 0: act = silu(gate) * up, or the clipped gate's product      KIND 1: act = relu(weight * up)^2      KIND 2: out (+)= scale * down
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 constexpr int kStageK = 32, kStagePitch = 40;
 
@@ -206,7 +212,7 @@ template <int KIND>
 __global__ __launch_bounds__(256) void moe_group_tiled_kernel(
     void* __restrict__ dst, int64_t ldo, const bf16_t* __restrict__ src, int64_t lds_rows, const bf16_t* __restrict__ w0,
     const bf16_t* __restrict__ w1, const int* __restrict__ order, const int* __restrict__ tiles, int most_tiles, int top,
-    int n_rows, int K, int add, const float* __restrict__ pair_weights, float weight) {
+    int n_rows, int K, int add, const float* __restrict__ pair_weights, float weight, int gate_act, GateNumbers numbers) {
   __shared__ __attribute__((aligned(16))) bf16_t As[2][kTilePairs * kStagePitch];
   __shared__ __attribute__((aligned(16))) bf16_t Ws[2][kTileRows * kStagePitch];
   if ((int)blockIdx.x >= tiles[3 * most_tiles]) return;
@@ -296,8 +302,8 @@ __global__ __launch_bounds__(256) void moe_group_tiled_kernel(
         bf16_t four[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float g = acc[0][j][4 * q + r];
-          four[r] = float_to_bf16(g / (1.0f + expf(-g)) * acc[1][j][4 * q + r]);
+          const float g = acc[0][j][4 * q + r], u = acc[1][j][4 * q + r];
+          four[r] = float_to_bf16(gate_act == GATE_CLIPPED ? clipped_gate(g, u, numbers) : g / (1.0f + expf(-g)) * u);
         }
         *reinterpret_cast<u32x2*>(o + f) = *reinterpret_cast<const u32x2*>(four);
       }
@@ -347,26 +353,30 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
 // with the same answer.  The sigmoid grows with its argument, so the largest scores are the largest logits.
 constexpr int kRouterMostExperts = 64 * 128;
 
-// score_kind 0: a score is sigmoid(z); 1: the softmax of z over all experts.  correction (float32 [experts] or
-// null) is added to a score where the experts are chosen and nowhere else: the weights are the scores.
+// score_kind 0: a score is sigmoid(z); 1: the softmax of z over all experts; 2: the softmax of z over the chosen
+// experts.  bias (float32 [experts] or null) is part of z.  correction (the same; not with kind 2) is added to a
+// score where the experts are chosen and nowhere else: the weights are the scores.
 __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restrict__ logits, int64_t ld, int n, int experts,
                                                           int top, int* __restrict__ chosen, float* __restrict__ weights,
-                                                          int score_kind, const float* __restrict__ correction) {
+                                                          int score_kind, const float* __restrict__ correction,
+                                                          const float* __restrict__ bias) {
   const int t = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= n) return;
-  const float* z = logits + (int64_t)t * ld;
+  const float* row = logits + (int64_t)t * ld;
+  auto z = [&](int e) { return bias != nullptr ? row[e] + bias[e] : row[e]; };
   float zmax = 0.f, inv_sum = 1.f;
   if (score_kind == 1) {
     zmax = -INFINITY;
-    for (int e = lane; e < experts; e += 64) zmax = fmaxf(zmax, z[e]);
+    for (int e = lane; e < experts; e += 64) zmax = fmaxf(zmax, z(e));
     zmax = wave_max(zmax);
     float sum = 0.f;
-    for (int e = lane; e < experts; e += 64) sum += expf(z[e] - zmax);
+    for (int e = lane; e < experts; e += 64) sum += expf(z(e) - zmax);
     inv_sum = 1.0f / wave_sum(sum);
   }
-  auto score = [&](int e) { return score_kind == 1 ? expf(z[e] - zmax) * inv_sum : 1.0f / (1.0f + expf(-z[e])); };
+  auto score = [&](int e) { return score_kind == 1 ? expf(z(e) - zmax) * inv_sum : 1.0f / (1.0f + expf(-z(e))); };
   // without a correction the order of the scores is the order of the logits (both scores grow with them)
-  auto choice = [&](int e) { return correction != nullptr ? score(e) + correction[e] : z[e]; };
+  auto choice = [&](int e) { return correction != nullptr ? score(e) + correction[e] : z(e); };
+  float first = 0.f, chosen_sum = 0.f;       // (kind 2: the largest logit, and the sum of the chosen ones' exponentials)
   unsigned long long taken[2] = {0ull, 0ull};
   for (int j = 0; j < top; ++j) {
     float best = -INFINITY;
@@ -384,20 +394,32 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
     if ((at & 63) == lane) taken[(at >> 6) >> 6] |= 1ull << ((at >> 6) & 63);
     if (lane == 0) {
       chosen[(int64_t)t * top + j] = at;
-      weights[(int64_t)t * top + j] = score(at);
+      if (score_kind == 2) {
+        if (j == 0) first = best;
+        const float w = expf(best - first);
+        chosen_sum += w;
+        weights[(int64_t)t * top + j] = w;
+      } else {
+        weights[(int64_t)t * top + j] = score(at);
+      }
     }
+  }
+  if (score_kind == 2 && lane == 0) {
+    const float inv = 1.0f / chosen_sum;
+    for (int j = 0; j < top; ++j) weights[(int64_t)t * top + j] *= inv;
   }
 }
 
 }  // namespace
 
 HFEE_API int hfee_router_topk(const float* logits, int64_t ld, int n, int experts, int top, int* chosen, float* weights,
-                              int score_kind, const float* correction, hipStream_t stream) {
-  HFEE_REQUIRE(score_kind == 0 || score_kind == 1, "router_topk: the scores are sigmoids (0) or a softmax (1)");
+                              int score_kind, const float* correction, const float* bias, hipStream_t stream) {
+  HFEE_REQUIRE(score_kind >= 0 && score_kind <= 2, "router_topk: the scores are sigmoids (0), a softmax (1) or a softmax over the chosen (2)");
+  HFEE_REQUIRE(score_kind != 2 || correction == nullptr, "router_topk: a softmax over the chosen experts takes no correction");
   HFEE_REQUIRE(n >= 0 && experts >= 1 && experts <= kRouterMostExperts && top >= 1 && top <= experts && ld >= experts,
                "router_topk: a token uses 1 to %d experts (of at most %d), not %d", experts, kRouterMostExperts, top);
   if (n == 0) return 0;
-  router_topk_kernel<<<(n + 3) / 4, 256, 0, stream>>>(logits, ld, n, experts, top, chosen, weights, score_kind, correction);
+  router_topk_kernel<<<(n + 3) / 4, 256, 0, stream>>>(logits, ld, n, experts, top, chosen, weights, score_kind, correction, bias);
   HFEE_CHECK_LAUNCH("router_topk");
   return 0;
 }
@@ -412,7 +434,10 @@ HFEE_API int hfee_moe_group_tiles(int n, int top, int experts) {
 HFEE_API int hfee_moe_grouped(float* x, int64_t ldx, const void* h, int64_t ldh, const void* w_gate, const void* w_up,
                               const void* w_down, const int* chosen, const int* table, const int* token_ids,
                               const float* pair_weights, float weight, int top, int experts, int ff, int width, int n,
-                              int* order, int* tiles, void* act, float* y, const float* in_weights, hipStream_t stream) {
+                              int* order, int* tiles, void* act, float* y, const float* in_weights, int gate_act, float limit,
+                              float sharpness, hipStream_t stream) {
+  HFEE_REQUIRE(gate_act == GATE_SILU || (gate_act == GATE_CLIPPED && w_gate != nullptr), "moe_grouped: unknown gate %d", gate_act);
+  const GateNumbers numbers{limit, sharpness};
   HFEE_REQUIRE(n >= 0 && top >= 1 && experts >= 1 && experts <= 8192 && ff >= 1 && width >= 1, "moe_grouped: bad sizes");
   HFEE_REQUIRE(chosen != nullptr || (table != nullptr && token_ids != nullptr), "moe_grouped: the experts of a token, or a table and the ids");
   HFEE_REQUIRE(width % 32 == 0 && ff % 32 == 0 && ldh % 8 == 0 && ldx >= width && ldh >= width,
@@ -430,14 +455,15 @@ HFEE_API int hfee_moe_grouped(float* x, int64_t ldx, const void* h, int64_t ldh,
   if (w_gate != nullptr)
     moe_group_tiled_kernel<0><<<dim3(most, (ff + kTileRows / 2 - 1) / (kTileRows / 2)), 256, 0, stream>>>(
         act, ff, (const bf16_t*)h, ldh, (const bf16_t*)w_gate, (const bf16_t*)w_up, order, tiles, most, top, ff, width, 0,
-        nullptr, 1.0f);
+        nullptr, 1.0f, gate_act, numbers);
   else
     moe_group_tiled_kernel<1><<<dim3(most, (ff + kTileRows - 1) / kTileRows), 256, 0, stream>>>(
-        act, ff, (const bf16_t*)h, ldh, (const bf16_t*)w_up, nullptr, order, tiles, most, top, ff, width, 0, in_weights, 1.0f);
+        act, ff, (const bf16_t*)h, ldh, (const bf16_t*)w_up, nullptr, order, tiles, most, top, ff, width, 0, in_weights, 1.0f,
+        GATE_SILU, numbers);
   HFEE_CHECK_LAUNCH("moe_group_up");
   moe_group_tiled_kernel<2><<<dim3(most, (width + kTileRows - 1) / kTileRows), 256, 0, stream>>>(
       top == 1 ? (void*)x : (void*)y, top == 1 ? ldx : (int64_t)width, (const bf16_t*)act, ff, (const bf16_t*)w_down, nullptr,
-      order, tiles, most, top, width, ff, top == 1 ? 1 : 0, pair_weights, weight);
+      order, tiles, most, top, width, ff, top == 1 ? 1 : 0, pair_weights, weight, GATE_SILU, numbers);
   HFEE_CHECK_LAUNCH("moe_group_down");
   if (top > 1) {
     int parts = (width + 255) / 256;
@@ -450,7 +476,10 @@ HFEE_API int hfee_moe_grouped(float* x, int64_t ldx, const void* h, int64_t ldh,
 
 HFEE_API int hfee_moe_up(void* act, const void* h, int64_t ldh, const void* w_gate, const void* w_up, int dtype,
                          const int* chosen, const int* table, const int* token_ids, int top, int experts, int ff,
-                         int width, int n, const float* in_weights, hipStream_t stream) {
+                         int width, int n, const float* in_weights, int gate_act, float limit, float sharpness,
+                         hipStream_t stream) {
+  HFEE_REQUIRE(gate_act == GATE_SILU || (gate_act == GATE_CLIPPED && w_gate != nullptr), "moe_up: unknown gate %d", gate_act);
+  const GateNumbers numbers{limit, sharpness};
   HFEE_REQUIRE(n >= 0 && top >= 1 && experts >= 1 && ff >= 1 && width >= 1 && ldh >= width, "moe_up: bad sizes");
   HFEE_REQUIRE(chosen != nullptr || (table != nullptr && token_ids != nullptr), "moe_up: the experts of a token, or a table and the ids");
   if (n == 0) return 0;
@@ -459,10 +488,12 @@ HFEE_API int hfee_moe_up(void* act, const void* h, int64_t ldh, const void* w_ga
   dim3 grid((unsigned)((int64_t)n * top), (ff + per_block - 1) / per_block);
   if (dtype == 0)
     moe_up_kernel<float><<<grid, 256, 0, stream>>>((float*)act, (const float*)h, ldh, (const float*)w_gate, (const float*)w_up,
-                                                   chosen, table, token_ids, top, experts, ff, width, in_weights);
+                                                   chosen, table, token_ids, top, experts, ff, width, in_weights,
+                                                    gate_act, numbers);
   else if (dtype == 1)
     moe_up_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)act, (const bf16_t*)h, ldh, (const bf16_t*)w_gate,
-                                                    (const bf16_t*)w_up, chosen, table, token_ids, top, experts, ff, width, in_weights);
+                                                    (const bf16_t*)w_up, chosen, table, token_ids, top, experts, ff, width, in_weights,
+                                                    gate_act, numbers);
   else
     return fail("moe_up: unknown dtype %d", dtype);
   HFEE_CHECK_LAUNCH("moe_up");

@@ -24,6 +24,7 @@ struct QkvArgs {
   int num_heads;
   // (the tiled kernels hand this struct to every epilogue: the gated one finds its activation here)
   int gate_act;               // GATE_SILU ...
+  GateNumbers gate_numbers;
 };
 
 

@@ -28,6 +28,7 @@
 //                       2  sigmoid(z)                                 (a writing strength)
 //                       3  z * factor for the first columns, z for the rest (a cast)
 //                       4  softplus(z + bias)                         (a step size)
+//                       5  silu(z + bias)                             (queries, keys and values behind a SiLU)
 //   rglru_scan          the real-gated linear recurrent unit, a number a channel:
 //                       a = exp(rate * sigmoid(r)), S <- a S + sqrt(1 - a^2) sigmoid(i) u, out = S * gelu(y + bias)
 //   gate_group_norm     out = norm((o + D[head] x) * silu(z)) * weight, the norm over each of `groups` equal parts
@@ -117,6 +118,7 @@ __global__ __launch_bounds__(256) void scan_gate_kernel(float* __restrict__ out,
   else if (mode == 1) r = expf(log_sigmoid(v) / number);
   else if (mode == 2) r = 1.0f / (1.0f + expf(-v));
   else if (mode == 4) r = softplus(v);
+  else if (mode == 5) r = v / (1.0f + expf(-v));
   else r = c < first_columns ? v * number : v;
   out[t * ldo + c] = r;
 }
@@ -361,6 +363,25 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(T* __restrict__ out
   for (int d = lane; d < V; d += 64) ss = fmaf(p[d], p[d], ss);
   const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)V + eps);
   for (int d = lane; d < V; d += 64) {
+    const float z = to_float<T>(gate[t * ldg + h * V + d]);
+    const float sig = 1.0f / (1.0f + expf(-z));
+    out[t * ldo + h * V + d] = from_float<T>(p[d] * inv * weight[d] * (act == 0 ? sig : z * sig));
+  }
+}
+
+// The same with a workgroup a (token, head), for heads of many values (all heads of a token normed together as one).
+template <typename T>
+__global__ __launch_bounds__(1024) void wide_head_norm_gate_kernel(T* __restrict__ out, int64_t ldo, const float* __restrict__ o,
+                                                                   int64_t ldi, const T* __restrict__ gate, int64_t ldg,
+                                                                   const float* __restrict__ weight, int heads, int V,
+                                                                   float eps, int act) {
+  __shared__ float scratch[16];
+  const int64_t t = blockIdx.x / heads, h = blockIdx.x % heads;
+  const float* p = o + t * ldi + h * V;
+  float ss = 0.f;
+  for (int d = threadIdx.x; d < V; d += blockDim.x) ss = fmaf(p[d], p[d], ss);
+  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)V + eps);
+  for (int d = threadIdx.x; d < V; d += blockDim.x) {
     const float z = to_float<T>(gate[t * ldg + h * V + d]);
     const float sig = 1.0f / (1.0f + expf(-z));
     out[t * ldo + h * V + d] = from_float<T>(p[d] * inv * weight[d] * (act == 0 ? sig : z * sig));
@@ -656,7 +677,7 @@ HFEE_API int hfee_scan_gate(float* out, int64_t ldo, const void* z, int64_t ldz,
                             const float* per_head, int head_width, int mode, float number, int first_columns, int n,
                             int width, hipStream_t stream) {
   HFEE_REQUIRE(n >= 0 && width > 0 && (width + 255) / 256 <= 65535 && ldo >= width && ldz >= width, "scan_gate: bad sizes");
-  HFEE_REQUIRE(mode >= 0 && mode <= 4, "scan_gate: unknown mode %d", mode);
+  HFEE_REQUIRE(mode >= 0 && mode <= 5, "scan_gate: unknown mode %d", mode);
   HFEE_REQUIRE(mode != 0 || (per_head != nullptr && head_width > 0), "scan_gate: a decay from a step size needs a number a head");
   HFEE_REQUIRE(mode != 1 || number > 0.f, "scan_gate: tau must be positive");
   if (n == 0) return 0;
@@ -711,6 +732,20 @@ HFEE_API int hfee_head_norm_gate(void* out, int64_t ldo, const float* o, int64_t
                "head_norm_gate: rows too short");
   if (n == 0) return 0;
   const int64_t items = (int64_t)n * heads;
+  HFEE_REQUIRE(items <= 0x7fffffff, "head_norm_gate: too much work for one launch");
+  if (vdim >= 1024) {
+    const int threads = n <= 64 ? 1024 : 256;
+    if (dtype == 0)
+      wide_head_norm_gate_kernel<float><<<(unsigned)items, threads, 0, stream>>>((float*)out, ldo, o, ldi, (const float*)gate,
+                                                                                ldg, weight, heads, vdim, eps, act);
+    else if (dtype == 1)
+      wide_head_norm_gate_kernel<bf16_t><<<(unsigned)items, threads, 0, stream>>>((bf16_t*)out, ldo, o, ldi, (const bf16_t*)gate,
+                                                                                 ldg, weight, heads, vdim, eps, act);
+    else
+      return fail("head_norm_gate: unknown dtype %d", dtype);
+    HFEE_CHECK_LAUNCH("head_norm_gate");
+    return 0;
+  }
   const unsigned blocks = (unsigned)((items + 3) / 4);
   if (dtype == 0)
     head_norm_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)out, ldo, o, ldi, (const float*)gate, ldg, weight,

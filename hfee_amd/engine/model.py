@@ -110,7 +110,7 @@ class Model:
         for layer, need in sorted(needs.items(), key=lambda kv: kv[0] if isinstance(kv[0], tuple) else (kv[0], 0)):
             by_need.setdefault(need, []).append(layer)
         return [CacheGroupSpec(kind=n.kind, token_shape=tuple(n.token_shape), window=n.window, layout=n.layout,
-                               every=n.every, cache_layers=tuple(layers))
+                               every=n.every, keep_first=n.keep_first, cache_layers=tuple(layers))
                 for n, layers in by_need.items()]
 
     def state_specs(self):

@@ -27,12 +27,12 @@ _CORE_SIGNATURES = {
     "hfee_embed_emit": [P, P, P, I, I, P, I, P, L, P, L, P],
     "hfee_rmsnorm": [P, I, P, P, I, P, F, I, I, P],
     "hfee_cast_rows": [P, I, P, P, I, I, P],
-    "hfee_swiglu": [P, L, P, P, L, I, I, I, I, I, P],
+    "hfee_swiglu": [P, L, P, P, L, I, I, I, I, I, F, F, P],
     "hfee_residual_add": [P, P, I, L, P],
     "hfee_rope_cache_write": [P, L, P, L, P, L, I, P, P, P, I, P, P, I, I, I, I, P, I, I, I, I, I, I, P],
     "hfee_gemm_f32": [P, L, P, L, P, L, I, I, I, I, P],
     "hfee_attention_ref": [P, L, P, L, P, I, P, P, P, I, I, I, I, I, F, I, I, P],
-    "hfee_gemm_bf16": [P, I, L, P, L, P, L, I, I, I, I, P, L, I, P],
+    "hfee_gemm_bf16": [P, I, L, P, L, P, L, I, I, I, I, P, L, I, F, F, P],
     "hfee_gemm_bf16_add_norm": [P, P, L, P, L, I, I, I, P, L, P, P, I, F, P],
     "hfee_gemm_bf16_cuts": [P, L, P, L, I, I, I, P, L, P, P],
     "hfee_rope_cache_write_cuts": [P, L, P, I, P, P, P, I, P, P, I, I, I, P, I, I, I, I, I, I, P],
@@ -48,7 +48,8 @@ _CORE_SIGNATURES = {
     "hfee_read_stream": [P, L, P, I, I, P],
     "hfee_mfma_loop": [P, I, I, P],
     "hfee_kv_write": [P, L, I, I, I, P, L, I, P, L, P, I, P, I, P, P, P, I, P, P, I, I, I, P, I, I, I, I, I, P],
-    "hfee_attention_kv_plain": [P, L, P, L, P, I, P, P, P, I, I, I, I, I, I, F, P, I, I, I, F, P, P, I, P, L, I, P],
+    "hfee_attention_kv_plain": [P, L, P, L, P, I, P, P, P, I, I, I, I, I, I, F, P, I, I, I, I, I, F, P, P, I, P, L, I, P],
+    "hfee_qkv_write": [P, L, P, L, I, P, L, P, L, I, P, P, P, I, P, P, F, P, P, I, I, I, P, P, P, I, P, I, I, I, I, I, P],
     "hfee_rotate_norm_write": [P, L, P, L, I, P, L, P, L, F, I, P, P, I, I, I, P, P, P, I, P, I, I, I, I, I, P],
     "hfee_kv_pool_write": [P, P, I, I, P, P, P, I, P, I, I, I, I, I, I, P],
     "hfee_rotate_rows": [P, L, P, L, I, P, P, P, I, I, I, I, I, I, F, I, P],
@@ -66,14 +67,17 @@ _CORE_SIGNATURES = {
     "hfee_linear_scan": [P, L, P, P, L, P, L, P, L, P, L, P, L, P, P, P, I, I, I, I, I, I, I, P],
     "hfee_rglru_scan": [P, L, I, P, P, L, P, P, L, P, P, L, P, P, P, P, I, I, I, I, P, L, P],
     "hfee_gate_group_norm": [P, L, I, P, L, P, L, P, I, P, L, P, I, I, F, I, P],
-    "hfee_router_topk": [P, L, I, I, I, P, P, I, P, P],
+    "hfee_router_topk": [P, L, I, I, I, P, P, I, P, P, P],
     "hfee_add_table_rows": [P, I, I, P, I, P, P],
     "hfee_scaled_add": [P, P, F, P, F, L, P],
     "hfee_scaled_add_norm": [P, P, F, P, I, P, F, I, I, P],
     "hfee_gated_norm_add": [P, P, P, F, F, P, I, L, P, P, F, P, I, P, F, I, I, P],
+    "hfee_post_norm": [P, P, F, P, F, F, P, F, P, I, P, P, P, I, I, P],
+    "hfee_token_shift": [P, I, P, P, P, P, P, P, P, I, I, P],
+    "hfee_softcap": [P, F, L, P],
     "hfee_head_norm_gate": [P, L, P, L, P, L, I, P, I, I, F, I, I, P],
-    "hfee_moe_grouped": [P, L, P, L, P, P, P, P, P, P, P, F, I, I, I, I, I, P, P, P, P, P, P],
-    "hfee_moe_up": [P, P, L, P, P, I, P, P, P, I, I, I, I, I, P, P],
+    "hfee_moe_grouped": [P, L, P, L, P, P, P, P, P, P, P, F, I, I, I, I, I, P, P, P, P, P, I, F, F, P],
+    "hfee_moe_up": [P, P, L, P, P, I, P, P, P, I, I, I, I, I, P, I, F, F, P],
     "hfee_moe_down": [P, L, P, P, I, P, P, P, P, F, I, I, I, I, I, I, P],
     "hfee_rmsnorm_cols": [P, L, P, L, I, P, I, F, F, I, I, P],
 }
@@ -83,7 +87,7 @@ _ATTENTION_KV_SIGNATURES = {
     "hfee_attention_kv_bf16_dv": [],
     "hfee_attention_kv_bf16_weights": [],
     "hfee_attention_kv_bf16_rows": [I],
-    "hfee_attention_kv_bf16": [P, L, P, L, P, P, I, I, P, I, I, I, I, F, P, P, L, I, I, I, F, P, P, I, P, L, P],
+    "hfee_attention_kv_bf16": [P, L, P, L, P, P, I, I, P, I, I, I, I, F, P, P, L, I, I, I, I, I, F, P, P, I, P, L, P],
 }
 
 _ATTENTION_MIX_SIGNATURES = {

@@ -138,7 +138,9 @@ def cast_rows(out: torch.Tensor, x: torch.Tensor, rows: torch.Tensor | None = No
 
 
 # the activations of a gated feed-forward's gate, as the kernels number them (GATE_SILU ... in csrc/common.h)
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "gelu": 2, "relu": 3}
+# ("clipped": not of the gate alone; with the numbers (limit, sharpness), g = min(gate, limit) and
+# u = clamp(up, -limit, limit), the product is g * sigmoid(sharpness * g) * (u + 1))
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "gelu": 2, "relu": 3, "clipped": 4}
 
 
 def gate_activation(name: str) -> int:
@@ -147,9 +149,18 @@ def gate_activation(name: str) -> int:
     return GATE_ACTIVATIONS[name]
 
 
-def swiglu(out: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, activation: str = "silu"):
+def gate_numbers(activation: str, numbers) -> tuple:
+    """(limit, sharpness) as the kernels take them: both needed by "clipped", zeros for the others."""
+    if activation != "clipped":
+        return 0.0, 0.0
+    _check(numbers is not None and len(numbers) == 2 and numbers[0] >= 0, "the clipped gate needs its limit and its sharpness")
+    return float(numbers[0]), float(numbers[1])
+
+
+def swiglu(out: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, activation: str = "silu", numbers=None):
     """out = activation(gate) * up ("silu": gate / (1 + exp(-gate))).  gate and up are views of one
-    buffer with the same row and column strides (column stride 1: two blocks; 2: alternating columns)."""
+    buffer with the same row and column strides (column stride 1: two blocks; 2: alternating columns).
+    "clipped" needs its `numbers` (limit, sharpness), see GATE_ACTIVATIONS."""
     act = gate_activation(activation)
     _gpu(out, gate, up)
     n, w, ldo = _rows2d(out, "swiglu out")
@@ -157,7 +168,8 @@ def swiglu(out: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, activation: 
     _check(gate.stride() == up.stride() and gate.stride(1) >= 1, "swiglu: gate and up must share their strides")
     _check(out.dtype == gate.dtype == up.dtype, "swiglu: dtype mismatch")
     ld = gate.stride(0) if n > 1 else max(gate.stride(0), (w - 1) * gate.stride(1) + 1)
-    lib.core().call("hfee_swiglu", _ptr(out), ldo, _ptr(gate), _ptr(up), ld, gate.stride(1), _dt(out), n, w, act, _stream())
+    lib.core().call("hfee_swiglu", _ptr(out), ldo, _ptr(gate), _ptr(up), ld, gate.stride(1), _dt(out), n, w, act,
+                    *gate_numbers(activation, numbers), _stream())
 
 
 def random_fill(out: torch.Tensor, key: int, kind: str, std: float = 1.0, bound: int = 0):
@@ -280,7 +292,7 @@ def linear_add_norm(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, no
 
 
 def linear(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, accumulate: bool = False, kernel: int = 0,
-           gate: bool = False, scratch=None, activation: str = "silu"):
+           gate: bool = False, scratch=None, activation: str = "silu", numbers=None):
     """out (+)= x @ weight.T, weight stored [out_features, in_features].
     scratch (bfloat16 products): float32, `linear_scratch(M, N, K)` words, or None.
 
@@ -288,7 +300,7 @@ def linear(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, accumulate:
     bfloat16 x and weight: matrix cores with float32 accumulation; out bfloat16, or
     float32 (required when accumulating: the residual stream).
     gate (bfloat16, aligned shapes): the rows of weight alternate gate/up and
-    out[m, j] = activation(row 2j) * row 2j+1, out [M, N/2].
+    out[m, j] = activation(row 2j) * row 2j+1, out [M, N/2] ("clipped" with its `numbers`, see GATE_ACTIVATIONS).
     kernel (bfloat16 only): 0 automatic, 1 skinny, 2 tiled 128x128, 3 the simple tiled
     kernel, 4 tiled 256x256, 5 tiled 256x128, 6 tiled 256x192, 7 and 8 tiled 128x128 and 128x192
     loaded straight into LDS."""
@@ -302,7 +314,7 @@ def linear(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, accumulate:
         _check(x.dtype == weight.dtype == out.dtype == torch.bfloat16 and not accumulate and N % 2 == 0,
                "linear: the gate epilogue takes bfloat16 operands and an even number of weight rows")
         lib.core().call("hfee_gemm_bf16", _ptr(out), 3, ldc, _ptr(x), lda, _ptr(weight), ldw, M, N, K, kernel,
-                        None, 0, gate_activation(activation), _stream())
+                        None, 0, gate_activation(activation), *gate_numbers(activation, numbers), _stream())
         return
     _check(x.dtype == weight.dtype, "linear: x and weight dtypes differ")
     if x.dtype == torch.float32:
@@ -320,7 +332,7 @@ def linear(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, accumulate:
             _gpu(scratch)
             _check(scratch.dtype == torch.float32 and scratch.is_contiguous(), "linear: float32 scratch expected")
         lib.core().call("hfee_gemm_bf16", _ptr(out), mode, ldc, _ptr(x), lda, _ptr(weight), ldw, M, N, K,
-                        kernel, _ptr(scratch), 0 if scratch is None else scratch.numel(), 0, _stream())
+                        kernel, _ptr(scratch), 0 if scratch is None else scratch.numel(), 0, 0.0, 0.0, _stream())
     else:
         raise KernelError(f"linear: unsupported dtype {x.dtype}")
 
@@ -849,10 +861,12 @@ def kv_write(q, k, v, positions, token_segment, block_tables, cos, sin, cache_la
 KEY_WEIGHTS = {"softmax": 0, "sigmoid": 1}
 
 
-def _sight(window: int, pool: int, softcap: float, pooled, pool_tables, cache_layer, segments: int, what: str):
+def _sight(window: int, pool: int, softcap: float, pooled, pool_tables, cache_layer, segments: int, what: str, chunk: int = 0,
+           keep_first: int = 0):
     """(the pooled layer, its block tables, their row stride) for the entry points; pooled blocks are a cache layer of
     the tokens' shape and dtype with block tables of its own, a row a segment."""
-    _check(window >= 0 and pool >= 0 and softcap >= 0, f"{what}: bad window, pool or softcap")
+    _check(window >= 0 and pool >= 0 and softcap >= 0 and chunk >= 0 and keep_first >= 0,
+           f"{what}: bad window, chunk, kept first keys, pool or softcap")
     if not (pool and window):
         return None, None, 0
     _check(pooled is not None and pool_tables is not None, f"{what}: pooled blocks need their cache layer and its block tables")
@@ -865,11 +879,14 @@ def _sight(window: int, pool: int, softcap: float, pooled, pool_tables, cache_la
 
 def attention_kv_plain(out, q, cache_layer, positions, token_segment, block_tables, num_heads: int, kv_heads: int,
                        dk: int, dv: int, page_size: int, scale: float, sinks=None, weights: str = "softmax",
-                       window: int = 0, pool: int = 0, softcap: float = 0.0, pooled=None, pool_tables=None, gate=None):
+                       window: int = 0, pool: int = 0, softcap: float = 0.0, pooled=None, pool_tables=None, gate=None,
+                       chunk: int = 0, keep_first: int = 0):
     """One wave per (token, head), any sizes, both dtypes: token t of head h reads the keys
     0..pos of its sequence; `sinks` (float32 [num_heads] or None) joins the softmax's denominator.
     weights "sigmoid": no softmax, a key weighs sigmoid(score + sinks[head]) and nothing is normalized.
-    window > 0: only the last `window` positions, the token's own included; pool > 0: also one key and
+    window > 0: only the last `window` positions, the token's own included; chunk > 0: only the positions of the
+    token's own chunk, position // chunk; keep_first: the first positions of the sequence that a window or a chunk
+    leaves in sight; pool > 0: also one key and
     value (entry b of the cache layer `pooled`, which has block tables of its own, `pool_tables`) for every
     block b of `pool` positions that lies wholly before the window; softcap > 0: a score s counts as
     softcap * tanh(s / softcap).
@@ -882,7 +899,7 @@ def attention_kv_plain(out, q, cache_layer, positions, token_segment, block_tabl
     _check(q.dtype == out.dtype == cache_layer.dtype, "attention_kv: dtype mismatch")
     _kv_cache(cache_layer, kv_heads, dk, dv, page_size, "attention_kv")
     pooled, pool_tables, pool_stride = _sight(window, pool, softcap, pooled, pool_tables, cache_layer, block_tables.shape[0],
-                                              "attention_kv")
+                                              "attention_kv", chunk, keep_first)
     _i32(positions, "attention_kv positions", n)
     _i32(token_segment, "attention_kv token_segment", n)
     _check(block_tables.dtype == torch.int32 and block_tables.dim() == 2 and block_tables.stride(1) == 1,
@@ -897,8 +914,8 @@ def attention_kv_plain(out, q, cache_layer, positions, token_segment, block_tabl
     lib.core().call("hfee_attention_kv_plain", _ptr(out), ldo, _ptr(q), ldq, _ptr(cache_layer), _dt(q),
                     _ptr(positions), _ptr(token_segment), _ptr(block_tables), block_tables.stride(0),
                     num_heads, kv_heads, dk, dv, page_size, float(scale), _ptr(sinks), KEY_WEIGHTS[weights],
-                    int(window), int(pool), float(softcap), _ptr(pooled), _ptr(pool_tables), pool_stride, _ptr(gate), ldg, n,
-                    _stream())
+                    int(window), int(chunk), int(keep_first), int(pool), float(softcap), _ptr(pooled), _ptr(pool_tables),
+                    pool_stride, _ptr(gate), ldg, n, _stream())
 
 
 def rotate_norm_write(q_out, q, k, v, positions, token_segment, block_tables, cos, sin, cache_layer, num_heads: int,
@@ -931,6 +948,55 @@ def rotate_norm_write(q_out, q, k, v, positions, token_segment, block_tables, co
     lib.core().call("hfee_rotate_norm_write", _ptr(q_out), ldqo, _ptr(q), ldq, num_heads, _ptr(k), ldk, _ptr(v), ldv,
                     -1.0 if value_eps is None else float(value_eps), _dt(q_out), _ptr(cos), _ptr(sin), half, table_positions,
                     int(max_position), _ptr(positions), _ptr(token_segment if has_k else None),
+                    _ptr(block_tables if has_k else None), block_tables.stride(0) if has_k else 0,
+                    _ptr(cache_layer if has_k else None), kv_heads, dk, dv, page_size, n, _stream())
+
+
+QK_NORMS = {None: 0, "head": 1, "row": 2}
+
+
+def qkv_write(q_out, q, k, v, positions, token_segment, block_tables, cos, sin, cache_layer, num_heads: int, kv_heads: int,
+              dk: int, dv: int, page_size: int, max_position: int, biases=(None, None, None), norm=None, q_weight=None,
+              k_weight=None, eps: float = 0.0):
+    """From the projections q [n, num_heads * dk], k, v (any leading dimensions, the cache's dtype): each plus its bias
+    (float32, one an element, or None); q and k with norm "head" divided by their root mean square over each head
+    and multiplied by a weight [dk], with "row" by that over all heads of the token and a weight of the row's width
+    (float32, or None for ones); the first 2 * half dims of a head rotated, pairs (i, i + half), cos/sin float32
+    [positions, half] or None.  q goes to q_out, k and v into the token's slot of `cache_layer`, everything in
+    float32 up to one rounding at the end.  k and v None: the queries only."""
+    _gpu(q_out, q, k, v, positions, token_segment, block_tables, cos, sin, cache_layer, q_weight, k_weight, *biases)
+    n, wq, ldq = _rows2d(q, "qkv_write q")
+    no, wo, ldqo = _rows2d(q_out, "qkv_write q_out")
+    _check(no == n and wq == wo == num_heads * dk and q_out.dtype == q.dtype and q_out.data_ptr() != q.data_ptr(),
+           "qkv_write: q and q_out of one shape and dtype, in two places")
+    _check(norm in QK_NORMS, f"qkv_write: the norm is one of {list(QK_NORMS)}")
+    _i32(positions, "qkv_write positions", n)
+    widths = (num_heads * dk, kv_heads * dk, kv_heads * dv)
+    for b, w in zip(biases, widths):
+        if b is not None:
+            _check(b.dtype == torch.float32 and b.is_contiguous() and b.numel() == w, "qkv_write: a bias is float32, one an element")
+    for w, row in ((q_weight, widths[0]), (k_weight, widths[1])):
+        if w is not None:
+            _check(norm is not None and w.dtype == torch.float32 and w.is_contiguous() and w.numel() == (row if norm == "row" else dk),
+                   "qkv_write: a norm's weight is float32, [dk] a head or one an element of the row")
+    ldk = ldv = 0
+    has_k = k is not None
+    if has_k:
+        nk, wk, ldk = _rows2d(k, "qkv_write k")
+        nv, wv, ldv = _rows2d(v, "qkv_write v")
+        _check(nk == nv == n and wk == widths[1] and wv == widths[2] and k.dtype == v.dtype == q.dtype == cache_layer.dtype,
+               "qkv_write: k/v shapes and dtypes")
+        _kv_cache(cache_layer, kv_heads, dk, dv, page_size, "qkv_write")
+        _i32(token_segment, "qkv_write token_segment", n)
+        _check(block_tables.dtype == torch.int32 and block_tables.dim() == 2 and block_tables.stride(1) == 1, "qkv_write: block tables")
+    half = table_positions = 0
+    if cos is not None:
+        _check(cos.shape == sin.shape and cos.dim() == 2 and cos.is_contiguous() and sin.is_contiguous()
+               and cos.dtype == sin.dtype == torch.float32, "qkv_write: cos/sin tables")
+        table_positions, half = cos.shape
+    lib.core().call("hfee_qkv_write", _ptr(q_out), ldqo, _ptr(q), ldq, num_heads, _ptr(k), ldk, _ptr(v), ldv, _dt(q),
+                    *[_ptr(b) for b in biases], QK_NORMS[norm], _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(cos), _ptr(sin),
+                    half, table_positions, int(max_position), _ptr(positions), _ptr(token_segment if has_k else None),
                     _ptr(block_tables if has_k else None), block_tables.stride(0) if has_k else 0,
                     _ptr(cache_layer if has_k else None), kv_heads, dk, dv, page_size, n, _stream())
 
@@ -1003,12 +1069,12 @@ def attention_kv_partial_words(num_items: int, num_heads: int, dv: int, splits: 
 def attention_kv_bf16(out, q, cache_layer, items, mode: int, block_tables, num_heads: int, kv_heads: int, dk: int,
                       dv: int, page_size: int, scale: float, sinks=None, partial=None, splits: int = 1,
                       weights: str = "softmax", window: int = 0, pool: int = 0, softcap: float = 0.0, pooled=None,
-                      pool_tables=None, gate=None):
+                      pool_tables=None, gate=None, chunk: int = 0, keep_first: int = 0):
     """Matrix-core attention, bfloat16 (weights: as in `attention_kv_plain`).  items: int32 [count, 4] on the device (first row, rows,
     first position, block-table row).  mode 0: an item is up to `attention_kv_rows` consecutive tokens of a portion;
     mode 1: an item is a single token (rows = 1), whose keys may be split over `splits` waves that
     leave partial results in `partial` (float32, `attention_kv_partial_words`) for a joining kernel.
-    window, pool, softcap, pooled, pool_tables, gate: as in `attention_kv_plain`."""
+    window, pool, softcap, pooled, pool_tables, gate, chunk, keep_first: as in `attention_kv_plain`."""
     _gpu(out, q, cache_layer, items, block_tables, sinks, partial, gate, pooled, pool_tables)
     n, w, ldq = _rows2d(q, "attention_kv q")
     no, wo, ldo = _rows2d(out, "attention_kv out")
@@ -1016,7 +1082,7 @@ def attention_kv_bf16(out, q, cache_layer, items, mode: int, block_tables, num_h
     _check(q.dtype == out.dtype == cache_layer.dtype == torch.bfloat16, "attention_kv: bfloat16 tensors expected")
     _kv_cache(cache_layer, kv_heads, dk, dv, page_size, "attention_kv")
     pooled, pool_tables, pool_stride = _sight(window, pool, softcap, pooled, pool_tables, cache_layer, block_tables.shape[0],
-                                              "attention_kv")
+                                              "attention_kv", chunk, keep_first)
     ldg = 0
     if gate is not None:
         ng, wg, ldg = _rows2d(gate, "attention_kv gate")
@@ -1033,8 +1099,8 @@ def attention_kv_bf16(out, q, cache_layer, items, mode: int, block_tables, num_h
     lib.attention_kv_bf16(dk, dv, weights).call(
         "hfee_attention_kv_bf16", _ptr(out), ldo, _ptr(q), ldq, _ptr(cache_layer), _ptr(items), items.shape[0], int(mode),
         _ptr(block_tables), block_tables.stride(0), num_heads, kv_heads, page_size, float(scale), _ptr(sinks),
-        _ptr(partial), 0 if partial is None else partial.numel(), int(splits), int(window), int(pool), float(softcap),
-        _ptr(pooled), _ptr(pool_tables), pool_stride, _ptr(gate), ldg, _stream())
+        _ptr(partial), 0 if partial is None else partial.numel(), int(splits), int(window), int(chunk), int(keep_first),
+        int(pool), float(softcap), _ptr(pooled), _ptr(pool_tables), pool_stride, _ptr(gate), ldg, _stream())
 
 
 def head_linear(out, x, weight, heads: int, n_in: int, n_out: int, tail: int = 0, x_head_stride: int | None = None,
@@ -1137,6 +1203,58 @@ def gated_norm_add(x, y, weight, eps: float, y2=None, scales=(1.0, 1.0), gate=No
     lib.core().call("hfee_gated_norm_add", _ptr(x), _ptr(y), _ptr(y2), float(scales[0]), float(scales[1]), _ptr(gate),
                     0 if gate is None else _dt(gate), ldg, _ptr(gate_bias), _ptr(weight), float(eps), _ptr(next_out),
                     0 if next_out is None else _dt(next_out), _ptr(next_weight), float(next_eps), n, d, _stream())
+
+
+def post_norm(x, y, alpha: float, weight, eps: float, scale: float = 1.0, y2=None, scale2: float = 1.0, next_out=None,
+              shift=None, state=None, segment_slots=None):
+    """With v = alpha * x + scale * y + scale2 * y2 (y2 optional): x (float32, the residual stream) <-
+    v / sqrt(mean(v^2) + eps) * weight; with next_out also the new row in next_out's dtype, or, given `shift` (float32
+    [d]), x_new + (before - x_new) * shift with `before` the row that state[slot] (float32 [slots, d]) holds, which
+    x_new then replaces: row r is the only token of segment r, slot = segment_slots[r].  y, y2 float32, contiguous."""
+    _gpu(x, y, y2, weight, next_out, shift, state, segment_slots)
+    n, d, _ = _rows2d(x, "post_norm x")
+    for t in (x, y, y2):
+        if t is not None:
+            _check(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (n, d), "post_norm: contiguous float32 rows of one shape")
+    _check(weight.dtype == torch.float32 and weight.is_contiguous() and weight.numel() == d, "post_norm: weight float32 [d]")
+    if next_out is not None:
+        _check(next_out.is_contiguous() and tuple(next_out.shape) == (n, d) and next_out.data_ptr() != x.data_ptr(), "post_norm: next_out")
+    if shift is not None:
+        _check(next_out is not None and shift.dtype == torch.float32 and shift.is_contiguous() and shift.numel() == d,
+               "post_norm: shift float32 [d], with next_out")
+        _check(state is not None and state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 2 and state.shape[1] == d,
+               "post_norm: state float32 [slots, d]")
+        _i32(segment_slots, "post_norm segment_slots", n)
+        _check(segment_slots.numel() == n, "post_norm: every row is a segment's only token")
+    lib.core().call("hfee_post_norm", _ptr(x), _ptr(y), float(scale), _ptr(y2), float(scale2), float(alpha), _ptr(weight), float(eps),
+                    _ptr(next_out), 0 if next_out is None else _dt(next_out), _ptr(shift),
+                    _ptr(state if shift is not None else None), _ptr(segment_slots if shift is not None else None), n, d, _stream())
+
+
+def token_shift(out, x, state, shift, token_segment, segment_rows, segment_lengths, segment_slots):
+    """out[t] = x[t] + (x[t - 1] - x[t]) * shift with x[t - 1] the row before in the same segment; before a segment's first
+    row stands state[slot] (float32 [slots, d]), which then gets the segment's last row.  x float32 [n, d],
+    contiguous; shift float32 [d]; out [n, d] in either dtype."""
+    _gpu(out, x, state, shift, token_segment, segment_rows, segment_lengths, segment_slots)
+    n, d, _ = _rows2d(x, "token_shift x")
+    _check(x.dtype == torch.float32 and x.is_contiguous() and out.is_contiguous() and tuple(out.shape) == (n, d), "token_shift: x and out")
+    _check(shift.dtype == torch.float32 and shift.is_contiguous() and shift.numel() == d, "token_shift: shift float32 [d]")
+    _check(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 2 and state.shape[1] == d,
+           "token_shift: state float32 [slots, d]")
+    segments = segment_rows.numel()
+    _i32(token_segment, "token_shift token_segment", n)
+    _i32(segment_rows, "token_shift segment_rows")
+    _i32(segment_lengths, "token_shift segment_lengths", segments)
+    _i32(segment_slots, "token_shift segment_slots", segments)
+    lib.core().call("hfee_token_shift", _ptr(out), _dt(out), _ptr(x), _ptr(state), _ptr(shift), _ptr(token_segment),
+                    _ptr(segment_rows), _ptr(segment_lengths), _ptr(segment_slots), n, d, _stream())
+
+
+def softcap(x, cap: float):
+    """x (float32, contiguous, in place) = cap * tanh(x / cap)."""
+    _gpu(x)
+    _check(x.dtype == torch.float32 and x.is_contiguous() and cap > 0, "softcap: contiguous float32 and a positive cap")
+    lib.core().call("hfee_softcap", _ptr(x), float(cap), x.numel(), _stream())
 
 
 def bias_act(out, x, bias, activation: str = "none", numbers=(0.0, 0.0)):
@@ -1393,14 +1511,15 @@ def rotate_rows(out, x, positions, cos, sin, heads: int, dim: int, max_position:
                     float(factor), n, _stream())
 
 
-SCAN_GATES = {"step_decay": 0, "root_sigmoid": 1, "sigmoid": 2, "cast": 3, "softplus": 4}
+SCAN_GATES = {"step_decay": 0, "root_sigmoid": 1, "sigmoid": 2, "cast": 3, "softplus": 4, "silu": 5}
 
 
 def scan_gate(out, z, kind: str, bias=None, per_head=None, head_width: int = 0, number: float = 1.0, first_columns: int = 0):
     """out (float32) from a projection z (engine dtype), column by column:
     "step_decay": exp(-exp(per_head[column // head_width]) * softplus(z + bias));
     "root_sigmoid": sigmoid(z + bias) ** (1 / number);  "sigmoid": sigmoid(z + bias);
-    "cast": z * number in the first `first_columns` columns, z in the others;  "softplus": softplus(z + bias)."""
+    "cast": z * number in the first `first_columns` columns, z in the others;  "softplus": softplus(z + bias);
+    "silu": silu(z + bias)."""
     _gpu(out, z, bias, per_head)
     n, w, ldz = _rows2d(z, "scan_gate z")
     no, wo, ldo = _f32rows(out, "scan_gate out")
@@ -1566,10 +1685,17 @@ def _in_weights(in_weights, w_gate, n, top, what):
                f"{what}: in_weights float32 [n, top]")
 
 
-def moe_up(act, h, w_gate, w_up, top: int, chosen=None, table=None, token_ids=None, in_weights=None):
+def _expert_gate(activation: str, numbers, w_gate, what):
+    _check(activation in ("silu", "clipped") and (activation == "silu" or w_gate is not None), f"{what}: experts' gates are 'silu' or 'clipped'")
+    return (GATE_ACTIVATIONS[activation], *gate_numbers(activation, numbers))
+
+
+def moe_up(act, h, w_gate, w_up, top: int, chosen=None, table=None, token_ids=None, in_weights=None, activation: str = "silu",
+           numbers=None):
     """act[t * top + j] = silu(w_gate[e] @ h[t]) * (w_up[e] @ h[t]), e the j-th expert of token t
     (chosen[t, j], or table[token_ids[t], j]); w_gate, w_up: [experts, ff, width].  w_gate None: experts
-    without a gate, act = relu(in_weights[t, j] * (w_up[e] @ h[t]))^2 (in_weights float32 or None for one)."""
+    without a gate, act = relu(in_weights[t, j] * (w_up[e] @ h[t]))^2 (in_weights float32 or None for one).
+    activation "clipped" with its `numbers` (limit, sharpness): the gate of that name in GATE_ACTIVATIONS."""
     _gpu(act, h, w_gate, w_up, chosen, table, token_ids, in_weights)
     n, width, ldh = _rows2d(h, "moe_up h")
     E, F, W = w_up.shape
@@ -1581,18 +1707,20 @@ def moe_up(act, h, w_gate, w_up, top: int, chosen=None, table=None, token_ids=No
     _experts_of(chosen, table, token_ids, n, top, "moe_up")
     _in_weights(in_weights, w_gate, n, top, "moe_up")
     lib.core().call("hfee_moe_up", _ptr(act), _ptr(h), ldh, _ptr(w_gate), _ptr(w_up), _dt(h), _ptr(chosen), _ptr(table),
-                    _ptr(token_ids), top, E, F, width, n, _ptr(in_weights), _stream())
+                    _ptr(token_ids), top, E, F, width, n, _ptr(in_weights), *_expert_gate(activation, numbers, w_gate, "moe_up"),
+                    _stream())
 
 
-ROUTER_SCORES = {"sigmoid": 0, "softmax": 1}
+ROUTER_SCORES = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}
 
 
-def router_topk(chosen, weights, logits, top: int, score: str = "sigmoid", correction=None):
+def router_topk(chosen, weights, logits, top: int, score: str = "sigmoid", correction=None, bias=None):
     """chosen (int32 [n, top]) = the experts with the `top` largest choice scores of each row of logits
     (float32 [n, experts]; of equal ones the lower number), weights (float32 [n, top]) their scores.  A score
     is sigmoid(logit), or with score "softmax" the softmax over the row; the choice score is the score plus
-    correction (float32 [experts]) where one is given, and the weights never hold it."""
-    _gpu(chosen, weights, logits, correction)
+    correction (float32 [experts]) where one is given, and the weights never hold it.  score "softmax_chosen": the
+    softmax over the chosen logits only.  bias (float32 [experts]) is added to the logits before everything else."""
+    _gpu(chosen, weights, logits, correction, bias)
     n, E, ld = _f32rows(logits, "router_topk logits")
     _check(score in ROUTER_SCORES, f"router_topk: the scores are {sorted(ROUTER_SCORES)}")
     _check(chosen.dtype == torch.int32 and chosen.is_contiguous() and tuple(chosen.shape) == (n, top), "router_topk: chosen int32 [n, top]")
@@ -1600,8 +1728,11 @@ def router_topk(chosen, weights, logits, top: int, score: str = "sigmoid", corre
     if correction is not None:
         _check(correction.dtype == torch.float32 and correction.is_contiguous() and correction.numel() == E,
                "router_topk: correction float32 [experts]")
+    _check(correction is None or score != "softmax_chosen", "router_topk: a softmax over the chosen experts takes no correction")
+    if bias is not None:
+        _check(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == E, "router_topk: bias float32 [experts]")
     lib.core().call("hfee_router_topk", _ptr(logits), ld, n, E, int(top), _ptr(chosen), _ptr(weights), ROUTER_SCORES[score],
-                    _ptr(correction), _stream())
+                    _ptr(correction), _ptr(bias), _stream())
 
 
 def moe_down(x, act, w_down, top: int, weight: float = 1.0, pair_weights=None, chosen=None, table=None, token_ids=None,
@@ -1634,12 +1765,13 @@ def moe_grouped_fits(dtype, width: int, ff: int) -> bool:
 
 
 def moe_grouped(x, h, w_gate, w_up, w_down, top: int, order, tiles, act, y=None, weight: float = 1.0, pair_weights=None,
-                chosen=None, table=None, token_ids=None, in_weights=None):
+                chosen=None, table=None, token_ids=None, in_weights=None, activation: str = "silu", numbers=None):
     """x[t] += sum_j weight_tj * w_down[e_j] @ (silu(w_gate[e_j] @ h[t]) * (w_up[e_j] @ h[t])), bfloat16, with the
     step's (token, expert) pairs grouped by expert on the device and multiplied in tiles on the matrix cores.
     order: int32 [n * top]; tiles: int32 [3 * moe_group_tiles(n, top, experts) + 1]; act: bfloat16
     [n * top, ff]; y: float32 [n * top, width] (where top > 1): scratch.  w_gate None: experts without a gate,
-    relu(in_weights[t, j] * (w_up[e_j] @ h[t]))^2 in the gate's place (then without pair_weights)."""
+    relu(in_weights[t, j] * (w_up[e_j] @ h[t]))^2 in the gate's place (then without pair_weights).  activation,
+    numbers: as in `moe_up`."""
     _gpu(x, h, w_gate, w_up, w_down, order, tiles, act, y, pair_weights, chosen, table, token_ids, in_weights)
     n, width, ldh = _rows2d(h, "moe_grouped h")
     nx, wx, ldx = _f32rows(x, "moe_grouped x")
@@ -1662,4 +1794,5 @@ def moe_grouped(x, h, w_gate, w_up, w_down, top: int, order, tiles, act, y=None,
     _experts_of(chosen, table, token_ids, n, top, "moe_grouped")
     lib.core().call("hfee_moe_grouped", _ptr(x), ldx, _ptr(h), ldh, _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(chosen),
                     _ptr(table), _ptr(token_ids), _ptr(pair_weights), float(weight), top, E, F, width, n, _ptr(order),
-                    _ptr(tiles), _ptr(act), _ptr(y), _ptr(in_weights), _stream())
+                    _ptr(tiles), _ptr(act), _ptr(y), _ptr(in_weights), *_expert_gate(activation, numbers, w_gate, "moe_grouped"),
+                    _stream())

@@ -10,7 +10,7 @@ from .mlp import DenseMLP, GatedMLP
 from .kv_attention import KvAttention, LatentAttention, SigmoidAttention, WindowAttention
 from .embedding import Embedding, Head
 from .mix_attention import MixedAttention
-from .recurrent import GatedDelta, GatedLinearAttention, RealGatedRecurrentUnit, Retention, StateSpace
+from .recurrent import GatedDelta, GatedLinearAttention, LightningAttention, RealGatedRecurrentUnit, Retention, StateSpace
 from .paired import SideBySide
 from .moe import RoutedMoE, TableMoE
-from .block import ParallelBlock, PreNormBlock, SandwichBlock
+from .block import ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock

@@ -14,6 +14,16 @@ the multiplication, the norm and the addition are one launch (`ops.gated_norm_ad
 second result with the two scales of a mixer that is two mixers side by side (what its `forward_into`
 returns).
 
+"postnorm" has its norms behind the additions: with the parameter `alpha`,
+x <- norm_a(alpha x + mixer(h)); x <- norm_b(alpha x + feed_forward(x)), h = x itself or, with the parameter
+`token_shift`, each token's x mixed with that of the token before it, h_t = x_t + (x_(t-1) - x_t) * mu element by
+element (mu a learned vector a layer; zeros before the first token; the last token's x is per-request state).
+A layer may have no feed-forward (then it ends behind norm_a).  The sub-layers write float32 rows; one launch adds
+them, norms the sum and makes the next sub-layer's input (`ops.post_norm`), across layers too; a mixer that is two
+side by side has its second rows and the two scales taken into that launch.  In a step of single tokens the token
+shift is part of the launch, in a step with portions a launch of its own (`ops.token_shift`: a portion's rows are
+the neighbours of rows that other workgroups make).
+
 "parallel" has one norm whose output both sub-layers read: with h = norm(x),
 x += mixer(h) + feed_forward(h).  Both add their last product straight into the float32 stream, the
 mixer first; a layer may have no feed-forward.  With the parameter `residual_scale` = m the layer adds
@@ -87,6 +97,19 @@ class PreNormBlock(Part):
             part.forward_add(ctx, x, h, *args, then=then)
         else:
             part.forward_add(ctx, x, h, *args)
+
+
+def rows_of(part, ctx, h, width, *args):
+    """A sub-layer's output as float32 rows (not yet added anywhere), and what its `forward_into`
+    returned: None, or dict(y2, scales) of a part whose result is scales[0] * rows + scales[1] * y2."""
+    y = ctx.rows("block.sublayer_rows", width, torch.float32)
+    second = None
+    if hasattr(part, "forward_into"):
+        second = part.forward_into(ctx, y, h if part.takes_lazy_norm else h.tensor(), *args)
+    else:           # a part that only knows how to add: into rows of zeros
+        y.zero_()
+        part.forward_add(ctx, y, h if part.takes_lazy_norm else h.tensor(), *args)
+    return y, second
 
 
 @register_block("sandwich")
@@ -163,19 +186,6 @@ class SandwichBlock(Part):
         return logits, bias
 
     @staticmethod
-    def _rows_of(part, ctx, h, width, *args):
-        """The sub-layer's output as float32 rows (not yet added anywhere), and what `forward_into`
-        returned: None, or dict(y2, scales) of a part whose result is scales[0] * rows + scales[1] * y2."""
-        y = ctx.rows("block.sublayer_rows", width, torch.float32)
-        second = None
-        if hasattr(part, "forward_into"):
-            second = part.forward_into(ctx, y, h if part.takes_lazy_norm else h.tensor(), *args)
-        else:           # a part that only knows how to add: into rows of zeros
-            y.zero_()
-            part.forward_add(ctx, y, h if part.takes_lazy_norm else h.tensor(), *args)
-        return y, second
-
-    @staticmethod
     def _add_normed(ctx, x, y, post_norm, bias, following, second=None, gate=None, gate_bias=None):
         """x += post_norm(y + bias), and the norm that follows in the same launch where it is of the
         same form and nobody has made it yet.  second / gate: see `ops.gated_norm_add`."""
@@ -206,16 +216,141 @@ class SandwichBlock(Part):
     def forward(self, ctx, x, entry, h_in=None, h_next=None):
         h = h_in if h_in is not None else self.begin(ctx, x)
         gate, gate_bias = self._gate_of(ctx, "mixer", h)
-        y, second = self._rows_of(self.mixer, ctx, h, self.hidden, entry.cache, entry.writes_cache)
+        y, second = rows_of(self.mixer, ctx, h, self.hidden, entry.cache, entry.writes_cache)
         if self.feed_forward is None:
             self._add_normed(ctx, x, y, self.mixer_post_norm, getattr(self.mixer, "output_bias", None), h_next, second, gate, gate_bias)
             return
         h2 = LazyNorm(ctx, self.feed_forward_norm, x)
         self._add_normed(ctx, x, y, self.mixer_post_norm, getattr(self.mixer, "output_bias", None), h2, second, gate, gate_bias)
         gate, gate_bias = self._gate_of(ctx, "feed_forward", h2)
-        y, second = self._rows_of(self.feed_forward, ctx, h2, self.hidden)
+        y, second = rows_of(self.feed_forward, ctx, h2, self.hidden)
         self._add_normed(ctx, x, y, self.feed_forward_post_norm, getattr(self.feed_forward, "output_bias", None), h_next,
                          second, gate, gate_bias)
+
+
+class _BlockInput(LazyNorm):
+    """What a sub-layer of a "postnorm" block reads: the stream itself in the engine's dtype or, with `shift` = (mu,
+    state), each token's row mixed with the row of the token before it.  `fill` makes it in the launch that
+    makes the stream's new rows, where it can."""
+
+    def __init__(self, ctx, x, shift=None):
+        super().__init__(ctx, None, x)
+        self.shift = shift
+
+    def _rows(self):
+        return self.ctx.rows("block.normed", self.x.shape[1])
+
+    def fill(self) -> dict:
+        """The arguments of `ops.post_norm` that make this input, which is then taken as made; {} where it
+        cannot be made there."""
+        if self._tensor is not None or (self.shift is None and self.ctx.dtype == self.x.dtype):
+            return {}
+        if self.shift is None:
+            self._tensor = self._rows()
+            return dict(next_out=self._tensor)
+        if self.ctx.n != len(self.ctx.segments):       # (portions: a row's neighbour is made by another workgroup)
+            return {}
+        self._tensor = self._rows()
+        mu, state = self.shift
+        return dict(next_out=self._tensor, shift=mu, state=state, segment_slots=self.ctx.segment_slots)
+
+    def tensor(self):
+        if self._tensor is None:
+            ctx = self.ctx
+            if self.shift is not None:
+                self._tensor = self._rows()
+                ops.token_shift(self._tensor, self.x, self.shift[1], self.shift[0], ctx.token_segment, ctx.segment_rows,
+                                ctx.segment_lengths, ctx.segment_slots)
+            elif ctx.dtype == self.x.dtype:
+                self._tensor = self.x
+            else:
+                self._tensor = self._rows()
+                ops.cast_rows(self._tensor, self.x)
+        return self._tensor
+
+
+@register_block("postnorm")
+class PostNormBlock(Part):
+    """Tensor names by role: mixer_norm, feed_forward_norm, token_shift (the whole name behind the layer's prefix), mixer
+    and feed_forward (prefixes)."""
+    graph_safe = True
+    chains_norms = True
+
+    def __init__(self, spec: LayerSpec, dtype: torch.dtype):
+        self.spec, self.dtype, self.hidden = spec, dtype, spec.hidden
+        self.alpha = float(spec.get("alpha", 1.0))
+        self.shifts = bool(spec.get("token_shift", False))
+
+        def norm(norm_spec, role):
+            made = lookup("norm", norm_spec.kind)(norm_spec, spec.name_of(role, role + ".weight"))
+            if getattr(made, "fused_form_f32", None) is None:
+                raise ValueError("a postnorm block norms its sums with v / sqrt(mean(v^2) + eps) * w")
+            return made
+        self.mixer_norm = norm(spec.mixer_norm, "mixer_norm")
+        self.mixer = lookup("mixer", spec.mixer.kind)(spec.mixer, spec.name_of("mixer", "mixer."), dtype)
+        self.feed_forward = self.feed_forward_norm = None
+        if spec.feed_forward is not None:
+            self.feed_forward_norm = norm(spec.feed_forward_norm, "feed_forward_norm")
+            self.feed_forward = lookup("feed_forward", spec.feed_forward.kind)(
+                spec.feed_forward, spec.name_of("feed_forward", "feed_forward."), dtype)
+        self.shift_name = spec.name_of("token_shift", "token_shift")
+        self.shift = None                    # (mu float32 [hidden], state [slots, hidden]), once prepared
+        self.mu = None
+
+    def _own(self):
+        return [p for p in (self.mixer_norm, self.mixer, self.feed_forward_norm, self.feed_forward) if p is not None]
+
+    def parts(self):
+        return [self] + [q for p in self._own() for q in p.parts()]
+
+    def cache_spec(self):
+        return self.mixer.cache_spec()
+
+    def key_layout(self):
+        return getattr(self.mixer, "key_layout", lambda: None)()
+
+    def tensor_specs(self):
+        specs = [s for p in self._own() for s in p.tensor_specs()]
+        if self.shifts:
+            specs.append(TensorSpec(self.shift_name, (self.hidden,), role="vector"))
+        return specs
+
+    def bind(self, tensors):
+        for p in self._own():
+            p.bind(tensors)
+            if getattr(p, "output_bias", None) is not None:
+                raise ValueError("a postnorm block's sub-layers have no bias behind their last product")
+        if self.shifts:
+            self.mu = tensors.pop(self.shift_name).to(torch.float32).contiguous()
+
+    def state_specs(self):
+        return [(self.shift_name + ".last", (self.hidden,), torch.float32)] if self.shifts else []
+
+    def prepare(self, info):
+        if self.shifts:
+            self.shift = (self.mu, info.storage.states[self.shift_name + ".last"])
+
+    def begin(self, ctx, x):
+        return _BlockInput(ctx, x, self.shift)
+
+    def _join(self, x, y, second, norm, following):
+        """x <- norm(alpha x + the sub-layer's result), and the input of what follows where that is a block like this."""
+        more = following.fill() if isinstance(following, _BlockInput) else {}
+        if second is not None:
+            more.update(scale=second["scales"][0], y2=second["y2"], scale2=second["scales"][1])
+        weight, eps = norm.fused_form_f32()
+        ops.post_norm(x, y, self.alpha, weight, eps, **more)
+
+    def forward(self, ctx, x, entry, h_in=None, h_next=None):
+        h = h_in if h_in is not None else self.begin(ctx, x)
+        y, second = rows_of(self.mixer, ctx, h, self.hidden, entry.cache, entry.writes_cache)
+        if self.feed_forward is None:
+            self._join(x, y, second, self.mixer_norm, h_next)
+            return
+        h2 = _BlockInput(ctx, x)
+        self._join(x, y, second, self.mixer_norm, h2)
+        y, second = rows_of(self.feed_forward, ctx, h2, self.hidden)
+        self._join(x, y, second, self.feed_forward_norm, h_next)
 
 
 @register_block("parallel")

@@ -5,7 +5,8 @@ Embedding: a row gather into the float32 residual stream, no scaling
 element is multiplied in float32 on its way; with `position_table` (a tensor name) and `positions` (its
 rows) a learned vector a position is added to the row, table[p] for a token at position p of its
 sequence, in float32 and not scaled.  Head: final norm and the
-vocabulary product only for the rows whose logits are wanted
+vocabulary product only for the rows whose logits are wanted, with the spec's `softcap` = c
+then c * tanh(logits / c)
 (/root/reference/internal/llm/forward.go:117-141); it shares the embedding table
 when the model has no separate head (/root/reference/internal/llm/model.go:118-121).
 """
@@ -72,6 +73,7 @@ class Head(Part):
     def __init__(self, spec: HeadSpec, norm, name, vocab: int, hidden: int, embedding, dtype: torch.dtype):
         self.norm, self.name, self.vocab, self.hidden = norm, name, vocab, hidden
         self.embedding, self.dtype = embedding, dtype
+        self.softcap = float(spec.get("softcap", 0.0) or 0.0)
         self.weight = None
 
     def parts(self):
@@ -97,6 +99,11 @@ class Head(Part):
 
     def forward(self, ctx, logits, x, rows):
         """logits[i] = head(norm(x[rows[i]])); logits float32 [len(rows), vocab]."""
+        self._product(ctx, logits, x, rows)
+        if self.softcap:
+            ops.softcap(logits, self.softcap)
+
+    def _product(self, ctx, logits, x, rows):
         w = logits.shape[0]
         fused = getattr(self.norm, "fused_form", lambda: None)()
         if self.streams and w <= ops.SKINNY_MAX_ROWS:

@@ -4,10 +4,17 @@
 key/value head h // (H/G)), key size Dk, value size Dv; q and k are rotated in the first
 `rotary_dim` dims of each head (the position part's tables carry the amplitude of a stretched
 rotation); score = q.k * scale over the keys up to the token's own position; the softmax may have a
-sink, one learned number a head that joins the denominator only (`sink`); the values may be blended
+sink that joins the denominator only (`sink`: "learned" or True, one number a head; "zero", the number 0); the values may be blended
 with those that the first blending layer of the model computed for the same token (`value_blend`:
 "source" keeps its values of the step for the layers behind it, "mix" writes
 (1 - t) v + t v_source with its own learned t, and the blended values are what the cache holds).
+With `bias` q, k and v each have one, added to their products; with `qk_norm` "head" q and k are divided by
+their root mean square over each head (eps `norm_eps`) and multiplied by a weight of the head's size that all
+heads share, with "row" by that over all heads of the token and a weight of the whole projection's size, in both
+cases before the rotation.  With `chunk` a query sees the positions of its own chunk, position // chunk, with
+`window` the last `window` positions, itself included; with `keep_first` it also sees the first so many tokens
+of its sequence.  The pages that a window or a chunk has passed go back to the cache manager, except those that
+hold the first tokens.
 
 "latent_attention": queries and keys/values through low-rank latents.  c_q = norm(W_dq h),
 q = W_uq c_q, laid out head by head as [plain dims | rotated dims]; W_dkv h gives the latent c
@@ -85,7 +92,8 @@ def plan_items(plan, rows: int) -> None:
 def attend(ctx, out, q, cache, tables, num_heads, kv_heads, dk, dv, scale, sinks, matrix: bool, weights: str = "softmax",
            sight=None, gate=None) -> None:
     """weights "sigmoid": no softmax, `sinks` holds the number a head that joins every score.  sight: None, or
-    dict(window, pool, softcap, pooled, pool_tables) of a mixer whose queries do not see every earlier key as it is."""
+    dict(window, chunk, keep_first, pool, softcap, pooled, pool_tables) of a mixer whose queries do not see every earlier
+    key as it is."""
     sight = sight or {}
     if not matrix:
         ops.attention_kv_plain(out, q, cache, ctx.positions, ctx.token_segment, tables, num_heads, kv_heads, dk, dv,
@@ -101,9 +109,10 @@ def attend(ctx, out, q, cache, tables, num_heads, kv_heads, dk, dv, scale, sinks
         # under a captured graph the split count is fixed for the whole width of the block table
         span = ctx.host.get("graph.max_context", ctx.host["attention_kv.single_max_position"] + 1)
         tiles = -(-span // _KEY_TILE)
-        if sight.get("window"):        # the window's tiles, and those of the pooled blocks before it
+        reach = min((r for r in (sight.get("window"), sight.get("chunk")) if r), default=0)
+        if reach:                      # the tiles of the window or chunk, of the kept first tokens and of the pooled blocks
             pooled = span // sight["pool"] if sight.get("pool") else 0
-            tiles = min(tiles, -(-sight["window"] // _KEY_TILE) + 1 + -(-pooled // _KEY_TILE))
+            tiles = min(tiles, -(-reach // _KEY_TILE) + 1 + -(-sight.get("keep_first", 0) // _KEY_TILE) + -(-pooled // _KEY_TILE))
         units = kv_heads * -(-(num_heads // kv_heads) // _ROWS)
         # (a split walks four tiles at least of keys and values of 256 dims together, and fewer of larger ones)
         splits = max(1, min(tiles // max(1, 1024 // (dk + dv)), _WAVES_WANTED // (count * units), _MOST_SPLITS))
@@ -175,7 +184,23 @@ class KvAttention(_KvMixer):
         self.dk = spec.get("key_dim")
         self.dv = spec.get("value_dim", self.dk)
         self.scale = float(spec.get("scale", self.dk ** -0.5))
-        self.has_sink = bool(spec.get("sink", False))
+        sink = spec.get("sink", False)
+        self.sink = "learned" if sink is True else sink or None       # None | "learned" | "zero"
+        if self.sink not in (None, "learned", "zero"):
+            raise ValueError(f"sink is False, 'learned' or 'zero', not {sink!r}")
+        self.has_bias = bool(spec.get("bias", False))
+        self.qk_norm, self.norm_eps = spec.get("qk_norm"), float(spec.get("norm_eps", 1e-6))
+        if self.qk_norm not in (None, "head", "row"):
+            raise ValueError(f"qk_norm is None, 'head' or 'row', not {self.qk_norm!r}")
+        self.window, self.chunk = int(spec.get("window", 0) or 0), int(spec.get("chunk", 0) or 0)
+        self.keep_first = int(spec.get("keep_first", 0) or 0)
+        if min(self.window, self.chunk, self.keep_first) < 0:
+            raise ValueError("window, chunk and keep_first are not negative")
+        reach = [r for r in (self.window, self.chunk) if r]
+        self.reach = min(reach) if reach else 0       # positions that a query sees at most, the kept first ones apart
+        if not self.reach:
+            self.keep_first = 0                # (nothing is ever out of sight)
+        self.sight = dict(window=self.window, chunk=self.chunk, keep_first=self.keep_first) if self.reach else None
         self.blend = spec.get("value_blend")              # None | "source" | "mix"
         if self.blend not in (None, "source", "mix"):
             raise ValueError(f"value_blend is None, 'source' or 'mix', not {self.blend!r}")
@@ -184,8 +209,13 @@ class KvAttention(_KvMixer):
         self.position = lookup("position", spec.position.kind)(spec.position) if spec.position else None
         if self.position is not None and self.position.pairing != 0:
             raise ValueError("kv_attention rotates pairs (i, i + half)")
+        self.prepares = self.has_bias or self.qk_norm is not None       # (more than a rotation stands before the cache)
+        if self.prepares and self.blend is not None:
+            raise ValueError("values are blended as they are projected: no bias or norm beside value_blend")
         self.names = self._names(spec, dict(q="q_proj.weight", k="k_proj.weight", v="v_proj.weight", o="o_proj.weight",
-                                            sink="sinks", value_blend="value_blend"))
+                                            q_bias="q_proj.bias", k_bias="k_proj.bias", v_bias="v_proj.bias",
+                                            q_norm="q_norm.weight", k_norm="k_norm.weight", sink="sinks",
+                                            value_blend="value_blend"))
         self.q_width, self.k_width, self.v_width = self.num_heads * self.dk, self.kv_heads * self.dk, self.kv_heads * self.dv
         self.out_width = self.num_heads * self.dv
         self.kernel_sizes = (self.dk, self.dv, self.num_heads // self.kv_heads)
@@ -195,27 +225,44 @@ class KvAttention(_KvMixer):
         n = self.names
         specs = [TensorSpec(n["q"], (self.q_width, self.hidden)), TensorSpec(n["k"], (self.k_width, self.hidden)),
                  TensorSpec(n["v"], (self.v_width, self.hidden)), TensorSpec(n["o"], (self.hidden, self.out_width))]
-        if self.has_sink:
+        if self.sink == "learned":
             specs.append(TensorSpec(n["sink"], (self.num_heads,), role="vector"))
-        # (a layer that blends nothing may still carry the number in its checkpoint)
-        specs.append(TensorSpec(n["value_blend"], (), role="vector", optional=self.blend != "mix"))
+        if self.has_bias:
+            specs += [TensorSpec(n["q_bias"], (self.q_width,), role="vector"), TensorSpec(n["k_bias"], (self.k_width,), role="vector"),
+                      TensorSpec(n["v_bias"], (self.v_width,), role="vector")]
+        if self.qk_norm is not None:
+            q, k = (self.dk, self.dk) if self.qk_norm == "head" else (self.q_width, self.k_width)
+            specs += [TensorSpec(n["q_norm"], (q,), role="vector", init=("one_plus_normal",)),
+                      TensorSpec(n["k_norm"], (k,), role="vector", init=("one_plus_normal",))]
+        if not self.prepares:      # (a layer that blends nothing may still carry the number in its checkpoint)
+            specs.append(TensorSpec(n["value_blend"], (), role="vector", optional=self.blend != "mix"))
         return specs
 
     def bind(self, tensors):
         n = self.names
         self.w_qkv = torch.cat([tensors.pop(n["q"]), tensors.pop(n["k"]), tensors.pop(n["v"])], dim=0).contiguous()
         self.w_o = tensors.pop(n["o"]).contiguous()
-        self.sinks = tensors.pop(n["sink"]).to(torch.float32).contiguous() if self.has_sink else None
+        self.sinks = None
+        if self.sink == "learned":
+            self.sinks = tensors.pop(n["sink"]).to(torch.float32).contiguous()
+        elif self.sink == "zero":
+            self.sinks = torch.zeros(self.num_heads, dtype=torch.float32, device=self.w_o.device)
+        f32 = lambda role: tensors.pop(n[role]).to(torch.float32).contiguous()      # noqa: E731
+        self.biases = tuple(f32(r) for r in ("q_bias", "k_bias", "v_bias")) if self.has_bias else (None, None, None)
+        self.q_norm, self.k_norm = (f32("q_norm"), f32("k_norm")) if self.qk_norm is not None else (None, None)
         t = tensors.pop(n["value_blend"], None)
         self.blend_weight = t.reshape(1).to(self.dtype).contiguous() if (t is not None and self.blend == "mix") else None
         self.w_qkv_tiles, self.w_o_tiles = tiles_of(self.dtype, self.w_qkv, self.w_o)
 
     def cache_spec(self):
-        return CacheNeed("full", (self.kv_heads, self.dk + self.dv), 0, layout=_LAYOUT)
+        # (a chunk's first position lies at most `chunk` - 1 before any of its queries, as a window's does)
+        return CacheNeed("window" if self.reach else "full", (self.kv_heads, self.dk + self.dv), self.reach, layout=_LAYOUT,
+                         keep_first=self.keep_first)
 
     def key_layout(self):
         pos = self.position
-        return (self.kv_heads, self.dk, self.dv, None if pos is None else pos.signature())
+        made = (self.qk_norm, self.norm_eps if self.qk_norm else None, self.has_bias) if self.prepares else ()
+        return (self.kv_heads, self.dk, self.dv, None if pos is None else pos.signature(), *made)
 
     def forward_into(self, ctx, out, h, cache_layer: int, writes_cache: bool):
         n = ctx.n
@@ -234,14 +281,24 @@ class KvAttention(_KvMixer):
         else:       # this run of the layer reads keys and values that another run wrote
             ops.linear(q, hn, self.w_qkv[:self.q_width])
             k = v = None
+        if self.prepares:
+            made = ctx.rows("kv_attention.q", self.q_width)
+            ops.qkv_write(made, q, k, v, ctx.positions, ctx.token_segment, tables, cos, sin, cache, H, G, dk, dv, ctx.page_size,
+                          ctx.max_position, biases=self.biases, norm=self.qk_norm, q_weight=self.q_norm, k_weight=self.k_norm,
+                          eps=self.norm_eps)
+            return self._attend(ctx, out, made, cache, tables)
         first = None
         if self.blend is not None and writes_cache:       # the source's values of this step's tokens
             first = ctx.workspace.rows("kv_attention.blend_source", n, self.v_width, self.dtype)
         ops.kv_write(q, k, v, ctx.positions, ctx.token_segment, tables, cos, sin, cache, H, G, dk, dk, dv, ctx.page_size,
                      ctx.max_position, v_first=first, v_first_mode={None: 0, "source": 1, "mix": 2}[self.blend],
                      v_mix=self.blend_weight)
+        self._attend(ctx, out, q, cache, tables)
+
+    def _attend(self, ctx, out, q, cache, tables):
         att = ctx.rows("kv_attention.out", self.out_width)
-        attend(ctx, att, q, cache, tables, H, G, dk, dv, self.scale, self.sinks, self.matrix)
+        attend(ctx, att, q, cache, tables, self.num_heads, self.kv_heads, self.dk, self.dv, self.scale, self.sinks, self.matrix,
+               sight=self.sight)
         product(ctx, out, att, self.w_o, self.w_o_tiles)
 
 

@@ -1,10 +1,11 @@
 """The gated feed-forward (/root/reference/internal/llm/forward.go:110-114,
 /root/reference/internal/ggml/ops.go:159-165): down(activation(gate(h)) * up(h)), added to
 the residual stream; the reference's activation is the SiLU, and which one it is is a
-parameter of the part (`activation`: one of `ops.GATE_ACTIVATIONS`).  gate and up run as
+parameter of the part (`activation`: one of `ops.GATE_ACTIVATIONS`; "clipped", which acts on gate and up
+together, takes its two numbers from `numbers`).  gate and up run as
 one product over a weight whose rows alternate gate_j, up_j, so that the gate is the
 product's epilogue (and a step of at most 64 tokens folds the norm in front of it into
-the same launch).
+the same launch).  `forward_into` writes the result as float32 rows instead of adding it.
 
 "dense_mlp" is the feed-forward without a gate: down(activation(up(h) + b_up)) + b_down, the
 activation one of `ops.ROW_ACTIVATIONS` ("relu2": the square of relu; "xielu": with two learned numbers
@@ -36,20 +37,25 @@ class GatedMLP(FeedForward):
         if self.activation not in ops.GATE_ACTIVATIONS:
             raise ValueError(f"the gated feed-forward has the activations {sorted(ops.GATE_ACTIVATIONS)}, "
                              f"not {self.activation!r}")
+        self.numbers = spec.get("numbers")         # (limit, sharpness) of the clipped gate
+        ops.gate_numbers(self.activation, self.numbers)
         self.prefix, self.dtype = prefix, dtype
+        given = dict(spec.get("names") or ())
+        defaults = dict(gate="gate_proj.weight", up="up_proj.weight", down="down_proj.weight")
+        self.names = {role: prefix + given.get(role, default) for role, default in defaults.items()}
         self.w_gate_up = self.w_down = None
 
     def tensor_specs(self):
-        p = self.prefix
-        return [TensorSpec(p + "gate_proj.weight", (self.intermediate, self.hidden)),
-                TensorSpec(p + "up_proj.weight", (self.intermediate, self.hidden)),
-                TensorSpec(p + "down_proj.weight", (self.hidden, self.intermediate))]
+        n = self.names
+        return [TensorSpec(n["gate"], (self.intermediate, self.hidden)),
+                TensorSpec(n["up"], (self.intermediate, self.hidden)),
+                TensorSpec(n["down"], (self.hidden, self.intermediate))]
 
     def bind(self, tensors):
-        p = self.prefix
-        self.w_gate_up = torch.stack([tensors.pop(p + "gate_proj.weight"), tensors.pop(p + "up_proj.weight")],
+        n = self.names
+        self.w_gate_up = torch.stack([tensors.pop(n["gate"]), tensors.pop(n["up"])],
                                      dim=1).reshape(2 * self.intermediate, self.hidden).contiguous()
-        self.w_down = tensors.pop(p + "down_proj.weight").contiguous()
+        self.w_down = tensors.pop(n["down"]).contiguous()
         # a second copy in tiles for steps of up to 64 rows, whose products stream the weights
         self.aligned = self.dtype == torch.bfloat16 and self.hidden % 8 == 0 and self.intermediate % 8 == 0
         tiles = ops.tile_weights_if_room(self.w_gate_up, self.w_down) if self.aligned else None
@@ -59,6 +65,12 @@ class GatedMLP(FeedForward):
             self.second_half_rows = 0
 
     def forward_add(self, ctx, x, h, then=None):
+        self._run(ctx, x, h, then, add=True)
+
+    def forward_into(self, ctx, out, h):
+        self._run(ctx, out, h, None, add=False)
+
+    def _run(self, ctx, x, h, then, add: bool):
         F, n = self.intermediate, ctx.n
         act = ctx.rows("mlp.act", F)
         aligned = self.aligned
@@ -81,19 +93,19 @@ class GatedMLP(FeedForward):
             else:
                 ops.linear_fused(out, h.tensor() if lazy else h, w, epilogue, **ctx.workspace.product_scratch(n, w))
             if not silu:
-                ops.swiglu(act, out[:, 0::2], out[:, 1::2], activation=self.activation)
+                ops.swiglu(act, out[:, 0::2], out[:, 1::2], activation=self.activation, numbers=self.numbers)
             # the down projection adds into x and, if asked, begins the norm that follows
             emit = then.offer() if then is not None else None
-            ops.linear_fused(x, act, self.w_down_tiles, "add", emit=emit,
+            ops.linear_fused(x, act, self.w_down_tiles, "add" if add else "f32", emit=emit,
                              **ctx.workspace.product_scratch(n, self.w_down_tiles))
             return
         hn = h.tensor() if lazy else h
         if aligned:   # the gate in the product's epilogue
-            ops.linear(act, hn, self.w_gate_up, gate=True, activation=self.activation)
+            ops.linear(act, hn, self.w_gate_up, gate=True, activation=self.activation, numbers=self.numbers)
         else:
             gate_up = ctx.rows("mlp.gate_up", 2 * F)
             ops.linear(gate_up, hn, self.w_gate_up)
-            ops.swiglu(act, gate_up[:, 0::2], gate_up[:, 1::2], activation=self.activation)
+            ops.swiglu(act, gate_up[:, 0::2], gate_up[:, 1::2], activation=self.activation, numbers=self.numbers)
         # the down projection adds into x and, if asked, goes on with the norm that follows
         # (where its K is cut over workgroups: the kernel that adds the cuts up has the row at hand)
         cut = ctx.workspace.split_scratch(n, self.w_down)
@@ -101,7 +113,7 @@ class GatedMLP(FeedForward):
         if after:
             ops.linear_add_norm(x, act, self.w_down, after["out"], after["weight"], after["eps"], **cut)
         else:
-            ops.linear(x, act, self.w_down, accumulate=True, **cut)
+            ops.linear(x, act, self.w_down, accumulate=add, **cut)
 
 
 @register_feed_forward("dense_mlp")

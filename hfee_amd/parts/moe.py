@@ -18,16 +18,21 @@ Steps of many tokens go through the same grouped kernels as above, few tokens an
 Its parameters make other routed experts of it: `score` "softmax" takes the softmax of z over all experts as
 the scores; `correction` adds a learned number an expert to the scores where the experts are chosen, and only
 there; `activation` "silu" gives the experts a gate, down(silu(gate(h)) * up(h)); `weight_on` "output"
-multiplies an expert's output by its weight instead of its input.
+multiplies an expert's output by its weight instead of its input.  `score` "softmax_chosen" takes the softmax over the chosen
+logits only; `router_bias` adds a learned number an expert to the logits; `activation` "clipped" with its
+`numbers` (limit, sharpness) is the gate that clips both of its sides (`ops.GATE_ACTIVATIONS`); `shared` = (ff, numbers)
+stands an expert beside them (the same form, its own size and numbers, tensors under the name `shared`) that
+every token uses with weight one.
 """
 from __future__ import annotations
 
 import torch
 
-from ..config.specs import FeedForwardSpec
+from ..config.specs import FeedForwardSpec, params
 from ..kernels import ops
 from ..weights.spec import TensorSpec
 from .base import FeedForward, LazyNorm, register_feed_forward
+from .mlp import GatedMLP
 
 
 @register_feed_forward("table_moe")
@@ -93,8 +98,8 @@ class TableMoE(FeedForward):
 
 @register_feed_forward("routed_moe")
 class RoutedMoE(FeedForward):
-    """Tensor names by role: router ([experts, hidden]), correction ([experts]); expert (a format for the expert's
-    number), gate, up, down."""
+    """Tensor names by role: router ([experts, hidden]), router_bias, correction ([experts]); expert (a format for the
+    expert's number), shared (a prefix), gate, up, down."""
     graph_safe = True
 
     def __init__(self, spec: FeedForwardSpec, prefix: str, dtype: torch.dtype):
@@ -105,21 +110,36 @@ class RoutedMoE(FeedForward):
         self.activation, self.score = spec.get("activation", "relu2"), spec.get("score", "sigmoid")
         self.weight_on = spec.get("weight_on", "input")
         self.has_correction = bool(spec.get("correction", False))
-        if self.activation not in ("relu2", "silu") or self.score not in ops.ROUTER_SCORES:
-            raise ValueError("the routed experts' activation is 'relu2' (no gate) or 'silu' (gated), their scores "
+        self.has_router_bias = bool(spec.get("router_bias", False))
+        if self.activation not in ("relu2", "silu", "clipped") or self.score not in ops.ROUTER_SCORES:
+            raise ValueError("the routed experts' activation is 'relu2' (no gate), 'silu' or 'clipped' (gated), their scores "
                              f"one of {sorted(ops.ROUTER_SCORES)}")
-        self.gated = self.activation == "silu"
+        self.gated = self.activation != "relu2"
+        self.gate = dict(activation=self.activation, numbers=spec.get("numbers")) if self.gated else {}
+        if self.gated:
+            ops.gate_numbers(**self.gate)
         if self.weight_on != ("output" if self.gated else "input") or spec.get("renormalize", False):
             raise ValueError("the weights multiply the inputs of experts without a gate and the outputs of gated ones, "
-                             "and are not renormalized")
+                             "and are not renormalized (but by the softmax over the chosen)")
+        if self.has_correction and self.score == "softmax_chosen":
+            raise ValueError("a softmax over the chosen experts takes no correction")
         if not 1 <= self.top <= self.experts:
             raise ValueError(f"a token uses 1 to {self.experts} experts, not {self.top}")
         given = dict(spec.get("names") or ())
         self.expert_names = given.get("expert", "experts.{}.")
         self.roles = {r: given.get(r, d) for r, d in dict(gate="gate_proj.weight", up="up_proj.weight", down="down_proj.weight",
-                                                         router="router.weight", correction="router.correction").items()}
+                                                         router="router.weight", router_bias="router.bias",
+                                                         correction="router.correction", shared="shared_expert.").items()}
         self.output_bias = None
-        self.correction = None
+        self.correction = self.router_bias = None
+        self.shared = None
+        if spec.get("shared") is not None:
+            if not self.gated:
+                raise ValueError("an expert that every token uses is a gated one")
+            ff, numbers = spec.get("shared")
+            self.shared = GatedMLP(FeedForwardSpec("gated_mlp", params(
+                hidden=self.hidden, intermediate=ff, activation=self.activation, numbers=numbers,
+                names=tuple((r, self.roles[r]) for r in ("gate", "up", "down")))), prefix + self.roles["shared"], dtype)
 
     def _name(self, e: int, role: str) -> str:
         return self.prefix + self.expert_names.format(e) + self.roles[role]
@@ -134,6 +154,10 @@ class RoutedMoE(FeedForward):
         specs.append(TensorSpec(self.prefix + self.roles["router"], (self.experts, self.hidden)))
         if self.has_correction:
             specs.append(TensorSpec(self.prefix + self.roles["correction"], (self.experts,), role="vector"))
+        if self.has_router_bias:
+            specs.append(TensorSpec(self.prefix + self.roles["router_bias"], (self.experts,), role="vector"))
+        if self.shared is not None:
+            specs += self.shared.tensor_specs()
         return specs
 
     def bind(self, tensors):
@@ -144,6 +168,10 @@ class RoutedMoE(FeedForward):
         self.w_router = tensors.pop(self.prefix + self.roles["router"]).contiguous()
         if self.has_correction:
             self.correction = tensors.pop(self.prefix + self.roles["correction"]).to(torch.float32).contiguous()
+        if self.has_router_bias:
+            self.router_bias = tensors.pop(self.prefix + self.roles["router_bias"]).to(torch.float32).contiguous()
+        if self.shared is not None:
+            self.shared.bind(tensors)
 
     def _choose(self, ctx, hn):
         n, top = ctx.n, self.top
@@ -152,12 +180,15 @@ class RoutedMoE(FeedForward):
         ws = ctx.workspace
         chosen = ws.flat("routed_moe.chosen", ws.capacity * top, torch.int32)[:n * top].view(n, top)
         weights = ws.flat("routed_moe.weights", ws.capacity * top, torch.float32)[:n * top].view(n, top)
-        ops.router_topk(chosen, weights, logits, top, score=self.score, correction=self.correction)
+        ops.router_topk(chosen, weights, logits, top, score=self.score, correction=self.correction, bias=self.router_bias)
         return chosen, weights
 
     def _run(self, ctx, out, h, add: bool):
         hn = h.tensor() if isinstance(h, LazyNorm) else h
         n, top = ctx.n, self.top
+        if self.shared is not None:         # (its last product fills the rows, or adds to them; the experts' sum joins)
+            self.shared._run(ctx, out, hn, None, add=add)
+            add = True
         chosen, weights = self._choose(ctx, hn)
         # (gated experts: the weight meets the output; experts without a gate: the input)
         on_input = None if self.gated else weights
@@ -172,10 +203,10 @@ class RoutedMoE(FeedForward):
             if not add:
                 out.zero_()
             ops.moe_grouped(out, hn, self.w_gate, self.w_up, self.w_down, top, order, tiles, act, y, weight=1.0, chosen=chosen,
-                            in_weights=on_input, pair_weights=on_output)
+                            in_weights=on_input, pair_weights=on_output, **self.gate)
             return
         act = ctx.rows("table_moe.act", top * self.intermediate).view(n * top, self.intermediate)
-        ops.moe_up(act, hn, self.w_gate, self.w_up, top, chosen=chosen, in_weights=on_input)
+        ops.moe_up(act, hn, self.w_gate, self.w_up, top, chosen=chosen, in_weights=on_input, **self.gate)
         ops.moe_down(out, act, self.w_down, top, weight=1.0, pair_weights=on_output, chosen=chosen, accumulate=add)
 
     def forward_into(self, ctx, out, h):

@@ -1,7 +1,8 @@
 """RMSNorm (/root/reference/internal/ggml/ops.go:124-134): y = x / sqrt(mean(x^2) + eps) * w,
 the sum in float32, x the float32 residual stream, y in the engine's dtype (with the parameter
 `weight_offset` the stored weight lies around zero and the norm multiplies by offset + w: the sum
-is made once, in float32, when the weight is bound); "layernorm": y = (x - mean) / sqrt(variance + eps) * w
+is made once, in float32, when the weight is bound; with the parameter `one_number` the tensor is a
+single number for all coordinates, spread over a float32 row when it is bound); "layernorm": y = (x - mean) / sqrt(variance + eps) * w
 with the variance as the mean of the squared deviations and no bias; and "none" for a
 place where a model has no norm (the rows as they are, in the engine's dtype)."""
 from __future__ import annotations
@@ -21,14 +22,17 @@ class RMSNorm(Norm):
     def __init__(self, spec: NormSpec, name: str):
         self.width, self.eps, self.name = spec.width, spec.eps, name
         self.offset = float(dict(spec.params).get("weight_offset", 0.0))
+        self.one_number = bool(dict(spec.params).get("one_number", False))
         self.weight = None
 
     def tensor_specs(self):
-        return [TensorSpec(self.name, (self.width,), role="vector",
+        return [TensorSpec(self.name, () if self.one_number else (self.width,), role="vector",
                            init=("normal",) if self.offset else ("one_plus_normal",))]
 
     def bind(self, tensors):
         self.weight = tensors[self.name]
+        if self.one_number:
+            self.weight = self.weight.to(torch.float32).reshape(1).expand(self.width).contiguous()
         if self.offset:
             self.weight = (self.weight.to(torch.float32) + self.offset).contiguous()
 

@@ -25,6 +25,11 @@ position (the position part's pairs (i, i + half)), k is then multiplied by dim^
 S <- decay_h S + k v^T, o = S^T q, with one decay a head from the spec; each head's o is divided by its root
 mean square (eps `norm_eps`, no weight), the heads side by side times silu(W_g h); then the output product.
 
+"lightning_attention": the same recurrence without a rotation and without a scale, q = silu(W_q h), k = silu(W_k h)
+(`num_heads` heads of `dim`), v = silu(W_v h) (heads of `vdim`), one fixed decay a head from the spec; the heads of a
+token are divided together by their root mean square (eps `norm_eps`), times a weight [heads * vdim], times
+sigmoid(W_g h); then the output product.
+
 "state_space" (state-space duality): one product gives [z | x | B | C | dt] (z, x: `num_heads` heads of
 `vdim`; B, C: `groups` groups of `state`; dt a head).  x, B and C together pass a short causal convolution
 per channel with a bias and a SiLU.  dt = softplus(dt + dt_bias); per head (head h reads group
@@ -289,6 +294,71 @@ class Retention(_StateMixer):
                         decay_per_head=True)
         gated = ctx.rows("retention.out", self.v_width)
         ops.head_norm_gate(gated, o, proj[:, self.at_g:], self.norm_weight, H, V, self.norm_eps, "silu")
+        product(ctx, x, gated, self.w_o, self.w_o_tiles, add=add)
+
+
+@register_mixer("lightning_attention")
+class LightningAttention(_StateMixer):
+    """Tensor names by role: q, k, v, g, o (matrices), norm ([heads * vdim])."""
+
+    def __init__(self, spec: MixerSpec, prefix: str, dtype: torch.dtype):
+        self.prefix, self.dtype = prefix, dtype
+        self.hidden = spec.get("hidden")
+        self.heads = spec.get("num_heads")
+        self.dim, self.vdim = spec.get("dim"), spec.get("vdim")
+        self.decay = tuple(float(d) for d in spec.get("decay"))
+        self.norm_eps = float(spec.get("norm_eps", 1e-6))
+        if len(self.decay) != self.heads:
+            raise ValueError(f"{len(self.decay)} decays for {self.heads} heads")
+        self.names = self._names(spec, dict(q="q_proj.weight", k="k_proj.weight", v="v_proj.weight", g="g_proj.weight",
+                                            o="o_proj.weight", norm="norm.weight"))
+        self.qk_width, self.v_width = self.heads * self.dim, self.heads * self.vdim
+
+    def tensor_specs(self):
+        n = self.names
+        return [TensorSpec(n["q"], (self.qk_width, self.hidden)), TensorSpec(n["k"], (self.qk_width, self.hidden)),
+                TensorSpec(n["v"], (self.v_width, self.hidden)), TensorSpec(n["g"], (self.v_width, self.hidden)),
+                TensorSpec(n["o"], (self.hidden, self.v_width)),
+                TensorSpec(n["norm"], (self.v_width,), role="vector", init=("one_plus_normal",))]
+
+    def bind(self, tensors):
+        n = self.names
+        # one product for everything that reads the layer's input: [q | k | v | g]
+        self.w_in = torch.cat([tensors.pop(n[r]) for r in ("q", "k", "v", "g")], dim=0).contiguous()
+        self.at_v = 2 * self.qk_width
+        self.at_g = self.at_v + self.v_width
+        self.w_o = tensors.pop(n["o"]).contiguous()
+        self.norm_weight = tensors.pop(n["norm"]).to(torch.float32).contiguous()
+        self.decays = torch.tensor(self.decay, dtype=torch.float32, device=self.w_o.device)
+        self.w_in_tiles, self.w_o_tiles = tiles_of(self.dtype, self.w_in, self.w_o)
+
+    def state_specs(self):
+        return [(self.prefix + "state", (self.heads, *ops.scan_state_shape(self.dim, self.vdim)), torch.float32)]
+
+    def prepare(self, info):
+        self.state = info.storage.states[self.prefix + "state"]
+
+    def forward_add(self, ctx, x, h, cache_layer: int, writes_cache: bool):
+        self._run(ctx, x, h, add=True)
+
+    def forward_into(self, ctx, out, h, cache_layer: int, writes_cache: bool):
+        self._run(ctx, out, h, add=False)
+
+    def _run(self, ctx, x, h, add: bool):
+        hn = h.tensor() if isinstance(h, LazyNorm) else h
+        H, D, V = self.heads, self.dim, self.vdim
+        rows, lengths, slots = self._segments(ctx)
+        total = self.w_in.shape[0]
+        proj = ctx.rows("lightning.in", (total + 7) // 8 * 8)[:, :total]
+        product(ctx, proj, hn, self.w_in, self.w_in_tiles)
+        qkv = ctx.rows("lightning.qkv", self.at_g, torch.float32)
+        ops.scan_gate(qkv, proj[:, :self.at_g], "silu")
+        q, k, v = qkv[:, :self.qk_width], qkv[:, self.qk_width:self.at_v], qkv[:, self.at_v:]
+        o = ctx.rows("lightning.read", self.v_width, torch.float32)
+        ops.linear_scan(o, self.state, q, k, v, self.decays, None, rows, lengths, slots, H, H, D, V, "decay_add",
+                        decay_per_head=True)
+        gated = ctx.rows("lightning.out", self.v_width)
+        ops.head_norm_gate(gated, o, proj[:, self.at_g:], self.norm_weight, 1, self.v_width, self.norm_eps, "sigmoid")
         product(ctx, x, gated, self.w_o, self.w_o_tiles, add=add)
 
 
