@@ -88,6 +88,13 @@ SAPOSUN_SIZES = {
     "4096-wide": dict(width=4096, heads=32, kv_heads=8, dim=128, expert_ff=2048, q_rank=1536),
 }
 
+# The Medulorn design at the same two layer sizes, beside Saposun (the closest of the other designs: windowed
+# attention, a fixed-decay recurrence, routed gated experts): its layers go in turn through attention over chunks
+# of 1,536 keys and a pair of attention over a window of 1,024 keys that keeps the first four (heads and head size
+# of the Llama layer of that width) and lightning attention (Saposun's heads of the retention); every layer has
+# sixteen routed experts, two a token, and one of the same size that every token uses.
+MEDULORN_SIZES = SAPOSUN_SIZES
+
 CONTEXT = 8192
 PROMPT = 1024
 PREFILL = 2048
@@ -152,6 +159,13 @@ def parse(argv=None):
                     help="with --saposun: only this layer size")
     ap.add_argument("--saposun-design", choices=["both", "saposun", "sabezen"], default="both",
                     help="with --saposun: only one of the two designs (for profiling)")
+    ap.add_argument("--medulorn", action="store_true",
+                    help="the Medulorn design beside Saposun at equal layer sizes instead of the serving benchmark: its own "
+                    "JSON line, prefill of 2,048 tokens and decode at --batch")
+    ap.add_argument("--medulorn-size", choices=sorted(MEDULORN_SIZES), default=None,
+                    help="with --medulorn: only this layer size")
+    ap.add_argument("--medulorn-design", choices=["both", "medulorn", "saposun"], default="both",
+                    help="with --medulorn: only one of the two designs (for profiling)")
     ap.add_argument("--no-extra-points", action="store_true",
                     help="skip the other shapes and the longer context that the default run adds under `points`")
     return ap.parse_args(argv)
@@ -292,6 +306,23 @@ def saposun_config(size: dict, layers: int, vocab: int = 32000) -> dict:
             "max_positions": 4096, "layers": out}
 
 
+def medulorn_config(size: dict, layers: int, vocab: int = 32000) -> dict:
+    d, H, G, hd = size["width"], size["heads"], size["kv_heads"], size["dim"]
+    heads = d // 256
+    att = {"type": "attention", "mixer": {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "scale": hd ** -0.5,
+                                          "mask": {"size": 1536}, "rot": {"base": 500000.0, "dims": hd}}}
+    left = {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": 1024, "keep_first": 4},
+            "rot": {"base": 500000.0, "dims": hd, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    right = {"heads": heads, "dim": 128, "vdim": 256,
+             "decay": [1.0 - 2.0 ** (-5 - 3 * i / max(1, heads - 1)) for i in range(heads)]}
+    pair = {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 1.0, "right_scale": 1.0}}
+    moe = {"kind": "moe", "expert": {"ff": size["expert_ff"], "limit": 7.0}, "router": {"experts": 16, "top": 2},
+           "shared": {"ff": size["expert_ff"], "limit": 7.0}}
+    return {"architecture": "Medulorn", "vocab": vocab, "width": d, "norm": {"eps": 1e-5}, "embedding": {"scale": d ** 0.5},
+            "postln_alpha": 2.0, "logit_softcap": 30.0, "max_positions": 4096,
+            "layers": [dict((att, pair)[i % 2], mlp=moe) for i in range(layers)]}
+
+
 def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
     """Prefill of 2,048 tokens and decode at `batch` requests of 1,024-token prompts for any
     registered architecture: times, and the fractions of the HBM and matrix peaks by the bytes a
@@ -313,6 +344,9 @@ def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
     for ls in spec.layers:
         f = ls.feed_forward
         if f is not None and f.kind in ("table_moe", "routed_moe"):
+            if f.get("shared") is not None:      # (the expert that every token uses, before the others' prefix)
+                shared = ls.name_of("feed_forward", "") + dict(f.get("names")).get("shared")
+                used[shared] = read[shared] = 1.0
             used[ls.name_of("feed_forward", "")] = f.get("top") / f.get("experts")
             read[ls.name_of("feed_forward", "")] = min(1.0, batch * f.get("top") / f.get("experts"))
 
@@ -324,14 +358,14 @@ def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
     chunked_flops = 0.0         # attention over chunks: the keys that a prompt of PREFILL tokens sees
     state_bytes = sum(4 * int(np.prod(shape)) for _, shape, dt in model.state_specs() if dt == torch.float32)
     scan_flops_a_token = 0      # the recurrences' multiply-adds on the vector units, counted apart
-    windows = []                # (elements a token, window, pool) of the cache layers that are read through a window
+    windows = []                # (elements a token, window, pool, own keys, chunk) of the cache layers that are read in part
     mixers = [m for ls in spec.layers for m in ((ls.mixer.get("left"), ls.mixer.get("right"))
                                                 if ls.mixer.kind == "side_by_side" else (ls.mixer,))]
     for m in mixers:
         if m.kind == "mixed_attention":
             seen = sum(i % m.get("chunk") + 1 for i in range(PREFILL)) if m.get("chunk") else PREFILL * (PREFILL + 1) / 2
             chunked_flops += 2.0 * 2 * m.get("dim") * m.get("num_heads") * seen
-        elif m.kind in ("gated_delta", "gla", "retention"):
+        elif m.kind in ("gated_delta", "gla", "retention", "lightning_attention"):
             scan_flops_a_token += 2 * (4 if m.kind == "gated_delta" else 3) * m.get("num_heads") * m.get("dim") * m.get("vdim")
         elif m.kind == "state_space":
             scan_flops_a_token += 2 * 3 * m.get("num_heads") * m.get("state") * m.get("vdim")
@@ -339,6 +373,12 @@ def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
             scan_flops_a_token += 2 * 2 * m.get("width") * (m.get("width") // m.get("blocks"))
         if m.kind == "attention":
             attention_dims += 2 * m.get("head_dim") * m.get("num_heads")
+        elif m.kind == "kv_attention" and (m.get("window") or m.get("chunk")):
+            dims, w, c = m.get("key_dim") + m.get("value_dim"), m.get("window") or 0, m.get("chunk") or 0
+            kept = m.get("keep_first") or 0
+            seen = sum(i % c + 1 if c else min(i + 1, w) + min(kept, max(0, i + 1 - w)) for i in range(PREFILL))
+            chunked_flops += 2.0 * dims * m.get("num_heads") * seen
+            windows.append((dims * m.get("num_kv_heads"), w, 0, True, c))
         elif m.kind in ("kv_attention", "sigmoid_attention"):
             attention_dims += (m.get("key_dim") + m.get("value_dim")) * m.get("num_heads")
         elif m.kind in ("latent_attention", "window_attention"):
@@ -348,7 +388,7 @@ def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
                 w, p = m.get("window"), m.get("pool") or 0
                 seen = sum(min(i + 1, w) + ((i - w + 1) // p if p and i - w + 1 >= p else 0) for i in range(PREFILL))
                 chunked_flops += 2.0 * dims * seen
-                windows.append((dims // m.get("num_heads") * (m.get("num_kv_heads") or 1), w, p, m.get("own_keys", True)))
+                windows.append((dims // m.get("num_heads") * (m.get("num_kv_heads") or 1), w, p, m.get("own_keys", True), 0))
             else:
                 attention_dims += dims
     page_size, context = 16, 4096
@@ -388,8 +428,9 @@ def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
     if chunks:
         context_read = context_read % min(chunks) + 1
     step_bytes = weight_bytes + batch * context_read * bytes_per_token(engine.groups, torch.bfloat16) + 2 * batch * state_bytes
-    for elements, w, p, own in windows:      # (a layer behind a window reads the window and the pooled blocks, not the context;
-        reads = min(context_read, w) + (context_read / p if p else 0)      # one that reads another layer's keys has no cache layer)
+    for elements, w, p, own, c in windows:      # (a layer behind a window reads the window and the pooled blocks, not the context;
+        # one that reads another layer's keys has no cache layer; a layer over chunks reads the chunk so far)
+        reads = context_read % c + 1 if c else min(context_read, w) + (context_read / p if p else 0)
         pooled_entries = context_read / p if p else 0                    # (the pooled blocks' group is counted by its share already)
         step_bytes -= batch * 2 * elements * ((context_read + pooled_entries if own else 0) - reads)
     for r in list(sched.running):
@@ -463,6 +504,23 @@ def saposun_compare(args) -> dict:
             "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16", "layers": layers, "points": points}
 
 
+def medulorn_compare(args) -> dict:
+    import hfee_amd  # noqa: F401
+    layers = args.layers or 6
+    points = {}
+    for name, size in MEDULORN_SIZES.items():
+        if args.medulorn_size not in (None, name):
+            continue
+        for design, cj in (("medulorn", medulorn_config(size, layers)), ("saposun", saposun_config(size, layers))):
+            if args.medulorn_design not in ("both", design):
+                continue
+            print(f"[bench] {design} {name}, {layers} layers", file=sys.stderr, flush=True)
+            points[f"{design}_{name}"] = design_point(cj, args.batch, min(args.steps, 32), min(args.warmup, 4))
+    return {"metric": "Medulorn beside Saposun at equal layer sizes: prefill of 2,048 tokens, decode at batch %d and "
+                      "1,024-token prompts (bf16, random weights)" % args.batch,
+            "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16", "layers": layers, "points": points}
+
+
 def sabezen_compare(args) -> dict:
     import hfee_amd  # noqa: F401
     layers = args.layers or 6
@@ -486,6 +544,9 @@ def main(argv=None) -> int:
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")
         return 2
+    if args.medulorn:
+        print(json.dumps(medulorn_compare(args)), flush=True)
+        return 0
     if args.saposun:
         print(json.dumps(saposun_compare(args)), flush=True)
         return 0
