@@ -200,10 +200,11 @@ __global__ __launch_bounds__(kScanWaves * 64) void linear_scan_kernel(
     const float* __restrict__ k, int64_t ldk, const float* __restrict__ v, int64_t ldv, const float* __restrict__ decay,
     int64_t ldd, const float* __restrict__ beta, int64_t ldb, const int* __restrict__ segment_rows,
     const int* __restrict__ segment_lengths, const int* __restrict__ segment_slots, int heads, int qk_heads, int D, int V,
-    int decay_per_head) {
+    int decay_per_head, int skip_from) {
   typedef ScanShape<DPT> Sh;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int seg = blockIdx.z, h = blockIdx.y, tid = threadIdx.x;
+  if (skip_from > 0 && segment_lengths[seg] >= skip_from) return;       // (linear_chunks.hip has this portion)
   const int lane = tid & 63, wave = tid >> 6;
   const int part = lane & (kScanParts - 1), c = lane >> 4;
   const int block = blockIdx.x * kScanWaves + wave;                 // of four columns
@@ -694,11 +695,12 @@ HFEE_API int hfee_scan_gate(float* out, int64_t ldo, const void* z, int64_t ldz,
   return 0;
 }
 
+// skip_from > 0: portions of that many tokens and more are left alone.
 HFEE_API int hfee_linear_scan(float* out, int64_t ldo, float* state, const float* q, int64_t ldq, const float* k,
                               int64_t ldk, const float* v, int64_t ldv, const float* decay, int64_t ldd,
                               const float* beta, int64_t ldb, const int* segment_rows, const int* segment_lengths,
                               const int* segment_slots, int segments, int heads, int qk_heads, int dim, int vdim,
-                              int rule, int decay_per_head, hipStream_t stream) {
+                              int rule, int decay_per_head, int skip_from, hipStream_t stream) {
   HFEE_REQUIRE(segments >= 0 && segments <= 65535, "linear_scan: bad segment count");
   if (segments == 0) return 0;
   HFEE_REQUIRE(heads > 0 && qk_heads > 0 && heads % qk_heads == 0 && heads <= 65535,
@@ -713,7 +715,7 @@ HFEE_API int hfee_linear_scan(float* out, int64_t ldo, float* state, const float
   const int per = (dim + kScanParts - 1) / kScanParts;
 #define LAUNCH(DPT, RULE)                                                                                             \
   linear_scan_kernel<DPT, RULE><<<grid, kScanWaves * 64, 2 * ScanShape<DPT>::BUFFER * sizeof(float), stream>>>(out, ldo, state, q, ldq, k, ldk, v, ldv, decay, ldd, beta, ldb, \
-      segment_rows, segment_lengths, segment_slots, heads, qk_heads, dim, vdim, decay_per_head)
+      segment_rows, segment_lengths, segment_slots, heads, qk_heads, dim, vdim, decay_per_head, skip_from)
 #define PICK(RULE)                                                                                                    \
   if (per <= 1) LAUNCH(1, RULE); else if (per <= 2) LAUNCH(2, RULE); else if (per <= 4) LAUNCH(4, RULE);              \
   else if (per <= 8) LAUNCH(8, RULE); else if (per <= 16) LAUNCH(16, RULE); else LAUNCH(32, RULE)

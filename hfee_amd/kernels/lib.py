@@ -64,7 +64,9 @@ _CORE_SIGNATURES = {
     "hfee_short_conv_keep": [P, P, L, I, P, P, P, I, I, I, P, P],
     "hfee_unit_heads": [P, L, I, I, F, F, I, P],
     "hfee_scan_gate": [P, L, P, L, I, P, P, I, I, F, I, I, I, P],
-    "hfee_linear_scan": [P, L, P, P, L, P, L, P, L, P, L, P, L, P, P, P, I, I, I, I, I, I, I, P],
+    "hfee_linear_scan": [P, L, P, P, L, P, L, P, L, P, L, P, L, P, P, P, I, I, I, I, I, I, I, I, P],
+    "hfee_linear_chunks": [P, L, P, P, L, P, L, P, L, P, P, P, P, I, I, I, I, I, I, I, I, P, L, P],
+    "hfee_linear_chunks_least": [],
     "hfee_rglru_scan": [P, L, I, P, P, L, P, P, L, P, P, L, P, P, P, P, I, I, I, I, P, L, P],
     "hfee_gate_group_norm": [P, L, I, P, L, P, L, P, I, P, L, P, I, I, F, I, P],
     "hfee_router_topk": [P, L, I, I, I, P, P, I, P, P, P],

@@ -1555,14 +1555,34 @@ def scan_state_matrix(state: torch.Tensor, dim: int, vdim: int) -> torch.Tensor:
     return s.reshape(*s.shape[:-4], s.shape[-4] * s.shape[-3], s.shape[-2] * s.shape[-1])[..., :dim, :vdim]
 
 
+LINEAR_CHUNK = 64       # tokens a chunk of the kernels for long portions
+
+
+def linear_chunks_fit(dim: int) -> bool:
+    """Whether the kernels in chunks take this key size (else every portion is walked token by token)."""
+    return dim % 4 == 0 and 4 <= dim <= 256
+
+
+def linear_chunks_scratch(longest: int, rows: int, heads: int, dim: int) -> int:
+    """float32 words with which `linear_scan` walks the long portions of a step (the longest of `longest` tokens, `rows`
+    in all) of a recurrence with fixed decays in chunks; 0 where it has none."""
+    if not linear_chunks_fit(dim) or longest < int(lib.core().raw("hfee_linear_chunks_least")()):
+        return 0
+    return heads * rows * LINEAR_CHUNK
+
+
 def linear_scan(out, state, q, k, v, decay, beta, segment_rows, segment_lengths, segment_slots, heads: int,
-                qk_heads: int, dim: int, vdim: int, rule: str, decay_per_head: bool = False):
+                qk_heads: int, dim: int, vdim: int, rule: str, decay_per_head: bool = False, longest: int = 0,
+                shortest: int = 0, scratch=None):
     """Walks each segment's rows in order from state[slot] (float32 [slots, heads, `scan_state_shape`],
     updated in place: a head's matrix in blocks of four columns).  rule "decay_add": S <- diag(decay) S + k v^T; "delta": S <- diag(decay) S,
     S <- S + k (beta (v - S^T k))^T; "scaled_add": S <- diag(decay) S + k (beta v)^T; out = S^T q.
     q, k: float32 [n, qk_heads * dim] (head h reads q/k head h // (heads / qk_heads)); v, out:
     [n, heads * vdim]; decay: [n, heads * dim], or with decay_per_head [n, heads], one number for all
-    of a head's rows (or [heads]: the same decays for every token); beta [n, heads]."""
+    of a head's rows (or [heads]: the same decays for every token); beta [n, heads].
+    With rule "decay_add" and the same decays for every token, `scratch` (float32, `linear_chunks_scratch` words) and
+    the lengths of the step's longest and shortest portion: long portions go in chunks through the matrix cores,
+    in float32 as well."""
     _gpu(out, state, q, k, v, decay, beta, segment_rows, segment_lengths, segment_slots)
     n, wq, ldq = _f32rows(q, "linear_scan q")
     nk, wk, ldk = _f32rows(k, "linear_scan k")
@@ -1587,9 +1607,22 @@ def linear_scan(out, state, q, k, v, decay, beta, segment_rows, segment_lengths,
     _i32(segment_rows, "linear_scan segment_rows")
     _i32(segment_lengths, "linear_scan segment_lengths", segments)
     _i32(segment_slots, "linear_scan segment_slots", segments)
+    skip_from = 0
+    if scratch is not None:
+        _gpu(scratch)
+        _check(rule == "decay_add" and decay.dim() == 1, "linear_scan: only fixed decays go in chunks")
+        _check(scratch.dtype == torch.float32 and scratch.is_contiguous() and 0 < shortest <= longest <= n, "linear_scan: scratch and lengths")
+        if ldq % 4 == 0 and ldk % 4 == 0 and q.data_ptr() % 16 == 0 and k.data_ptr() % 16 == 0:
+            skip_from = int(lib.core().raw("hfee_linear_chunks_least")())
+            lib.core().call("hfee_linear_chunks", _ptr(out), ldo, _ptr(state), _ptr(q), ldq, _ptr(k), ldk, _ptr(v), ldv, _ptr(decay),
+                            _ptr(segment_rows), _ptr(segment_lengths), _ptr(segment_slots), segments, int(longest), n, heads,
+                            qk_heads, dim, vdim, _scan_rows_a_lane(dim), _ptr(scratch), scratch.numel(), _stream())
+            if shortest >= skip_from:
+                return
     lib.core().call("hfee_linear_scan", _ptr(out), ldo, _ptr(state), _ptr(q), ldq, _ptr(k), ldk, _ptr(v), ldv, _ptr(decay),
                     ldd, _ptr(beta if rule != "decay_add" else None), ldb, _ptr(segment_rows), _ptr(segment_lengths),
-                    _ptr(segment_slots), segments, heads, qk_heads, dim, vdim, rules[rule], 1 if decay_per_head else 0, _stream())
+                    _ptr(segment_slots), segments, heads, qk_heads, dim, vdim, rules[rule], 1 if decay_per_head else 0, skip_from,
+                    _stream())
 
 
 RGLRU_CHUNK = 32        # tokens a chunk of the recurrent unit's kernels for long portions

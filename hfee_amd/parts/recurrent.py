@@ -69,6 +69,15 @@ class _StateMixer(Mixer):
     def _segments(self, ctx):
         return ctx.segment_rows, ctx.segment_lengths, ctx.segment_slots
 
+    @staticmethod
+    def _in_chunks(ctx, heads: int, dim: int) -> dict:
+        """The arguments with which `ops.linear_scan` walks a step's long portions in chunks (fixed decays only)."""
+        lengths = [s.length for s in ctx.segments]
+        words = ops.linear_chunks_scratch(max(lengths), ctx.n, heads, dim)
+        if not words:
+            return {}
+        return dict(scratch=ctx.workspace.flat("recurrent.chunks", words, torch.float32), longest=max(lengths), shortest=min(lengths))
+
 
 @register_mixer("gated_delta")
 class GatedDelta(_StateMixer):
@@ -291,7 +300,7 @@ class Retention(_StateMixer):
         q, k, v = qkv[:, :self.qk_width], qkv[:, self.qk_width:self.at_v], qkv[:, self.at_v:]
         o = ctx.rows("retention.read", self.v_width, torch.float32)
         ops.linear_scan(o, self.state, q, k, v, self.decays, None, rows, lengths, slots, H, H, D, V, "decay_add",
-                        decay_per_head=True)
+                        decay_per_head=True, **self._in_chunks(ctx, H, D))
         gated = ctx.rows("retention.out", self.v_width)
         ops.head_norm_gate(gated, o, proj[:, self.at_g:], self.norm_weight, H, V, self.norm_eps, "silu")
         product(ctx, x, gated, self.w_o, self.w_o_tiles, add=add)
@@ -356,7 +365,7 @@ class LightningAttention(_StateMixer):
         q, k, v = qkv[:, :self.qk_width], qkv[:, self.qk_width:self.at_v], qkv[:, self.at_v:]
         o = ctx.rows("lightning.read", self.v_width, torch.float32)
         ops.linear_scan(o, self.state, q, k, v, self.decays, None, rows, lengths, slots, H, H, D, V, "decay_add",
-                        decay_per_head=True)
+                        decay_per_head=True, **self._in_chunks(ctx, H, D))
         gated = ctx.rows("lightning.out", self.v_width)
         ops.head_norm_gate(gated, o, proj[:, self.at_g:], self.norm_weight, 1, self.v_width, self.norm_eps, "sigmoid")
         product(ctx, x, gated, self.w_o, self.w_o_tiles, add=add)

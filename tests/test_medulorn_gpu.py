@@ -257,10 +257,12 @@ def test_the_token_shift_across_portions(dtype, width):
     assert fed == lengths and torch.isnan(state[1]).all()
 
 
-@pytest.mark.parametrize("H,D,V", [(2, 16, 32), (3, 12, 20), (4, 64, 64), (1, 4, 4), (2, 128, 256)])
-def test_the_recurrence_in_portions(H, D, V):
-    """Two requests in other slots, in portions of unequal size, against the closed form
-    o_t = sum_j decay^(t - j) (q_t . k_j) v_j; a slot of NaNs beside them stays untouched."""
+@pytest.mark.parametrize("chunks", [False, True])
+@pytest.mark.parametrize("H,D,V", [(2, 16, 32), (3, 12, 20), (4, 64, 64), (1, 4, 4), (2, 128, 256), (3, 100, 17), (2, 256, 48)])
+def test_the_recurrence_in_portions(H, D, V, chunks):
+    """Two requests in other slots, in portions of unequal size, token by token and with the long portions in
+    chunks, against the closed form o_t = sum_j decay^(t - j) (q_t . k_j) v_j; a slot of NaNs beside them stays
+    untouched."""
     from hfee_amd.kernels import ops
     g = torch.Generator().manual_seed(H + D)
     lengths, slots = [290, 90], [2, 0]
@@ -282,8 +284,13 @@ def test_the_recurrence_in_portions(H, D, V):
         q, k, v = cat(qs), cat(ks), cat(vs)
         rows = np.cumsum([0] + [n for _, n in segs])[:-1]
         out = torch.zeros(q.shape[0], H * V, device="cuda")
+        more = {}
+        words = ops.linear_chunks_scratch(max(n for _, n in segs), q.shape[0], H, D)
+        if chunks and words:
+            more = dict(scratch=torch.full((words,), float("nan"), device="cuda"), longest=max(n for _, n in segs),
+                        shortest=min(n for _, n in segs))
         ops.linear_scan(out, state, q, k, v, decay.cuda(), None, i32(rows), i32([n for _, n in segs]), i32([slots[s] for s, _ in segs]),
-                        H, H, D, V, "decay_add", decay_per_head=True)
+                        H, H, D, V, "decay_add", decay_per_head=True, **more)
         row = 0
         for s, n in segs:
             assert mu.rel(out[row:row + n].double().cpu(), want[s][fed[s]:fed[s] + n]) < 2e-5, (sizes, s)
