@@ -271,6 +271,175 @@ __global__ __launch_bounds__(256) void qkv_write_kernel(
   }
 }
 
+// The same in bfloat16 for heads in whole groups of eight dims (rotated dims in sixteens) and rows of 16-byte pieces:
+// a thread takes up to R pieces of a row, each the eight pairs (d .. d + 7, d + half .. d + half + 7) of a head
+// or eight dims that are not rotated, and holds them from the sums to the stores.  Workgroups: first those that take
+// the values of 16 tokens each in parts of 256 columns (the cache holds values by column: 16 tokens that fill 16
+// slots in a row are 32 neighbouring bytes there, and one store), then a workgroup a token's queries, then a
+// workgroup a token's keys.  A head's sum of squares is added up over its pieces in their order.
+constexpr int kQkvValueColumns = 256, kQkvPieces = 4;
+
+// eight neighbouring float32 (32-byte aligned places), or eight times `otherwise` where there are none
+__device__ __forceinline__ void eight_floats(float (&o)[8], const float* p, float otherwise) {
+  float lo[4] = {otherwise, otherwise, otherwise, otherwise}, hi[4] = {otherwise, otherwise, otherwise, otherwise};
+  if (p != nullptr) {
+    load4<float>(lo, p);
+    load4<float>(hi, p + 4);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    o[i] = lo[i];
+    o[4 + i] = hi[i];
+  }
+}
+
+template <int NORM, int R>
+__global__ __launch_bounds__(256) void qkv_write_pieces_kernel(
+    bf16_t* __restrict__ q_out, int64_t ldqo, const bf16_t* __restrict__ q, int64_t ldq, int num_heads,
+    const bf16_t* __restrict__ k, int64_t ldk, const bf16_t* __restrict__ v, int64_t ldv, const float* __restrict__ q_bias,
+    const float* __restrict__ k_bias, const float* __restrict__ v_bias, const float* __restrict__ q_weight,
+    const float* __restrict__ k_weight, float eps, const float* __restrict__ cos_t, const float* __restrict__ sin_t, int half,
+    const int* __restrict__ positions, const int* __restrict__ token_segment, const int* __restrict__ block_tables,
+    int bt_stride, bf16_t* __restrict__ cache, KvLayout lay, int n, int value_groups, int value_parts) {
+  typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+  union Eight {
+    u32x4 u;
+    bf16_t e[8];
+  };
+  __shared__ float sums[R * 256];
+  __shared__ float scratch[16];
+  __shared__ __attribute__((aligned(16))) bf16_t columns[16][kQkvValueColumns + 8];
+  __shared__ int g_pos[16], g_seg[16], g_page[16];
+  const int tid = threadIdx.x;
+  int id = blockIdx.x;
+  if (id < value_groups * value_parts) {
+    const int t0 = id / value_parts * 16, c0 = id % value_parts * kQkvValueColumns;
+    const int count = min(16, n - t0), width = min(kQkvValueColumns, lay.kv_heads * lay.dv - c0), pieces = width / 8;
+    if (tid < count) {
+      const int p = positions[t0 + tid], s = token_segment[t0 + tid];
+      g_pos[tid] = p;
+      g_seg[tid] = s;
+      g_page[tid] = block_tables[(int64_t)s * bt_stride + (p >> lay.page_shift)];
+    }
+    for (int e = tid; e < count * pieces; e += blockDim.x) {
+      const int j = e / pieces, c = (e - j * pieces) * 8;
+      Eight x;
+      x.u = *reinterpret_cast<const u32x4*>(v + (int64_t)(t0 + j) * ldv + c0 + c);
+      if (v_bias != nullptr) {
+        float add[8];
+        eight_floats(add, v_bias + c0 + c, 0.f);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) x.e[i] = float_to_bf16(bf16_to_float(x.e[i]) + add[i]);
+      }
+      *reinterpret_cast<u32x4*>(&columns[j][c]) = x.u;
+    }
+    __syncthreads();
+    bool in_a_row = count == 16 && (g_pos[0] & 15) == 0;
+    for (int j = 1; j < count; ++j) in_a_row = in_a_row && g_pos[j] == g_pos[0] + j && g_seg[j] == g_seg[0];
+    for (int c = tid; c < width; c += blockDim.x) {
+      const int g = (c0 + c) / lay.dv, d = (c0 + c) - g * lay.dv;
+      if (in_a_row) {
+        Eight lo, hi;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          lo.e[j] = finite_bf16(columns[j][c]);
+          hi.e[j] = finite_bf16(columns[8 + j][c]);
+        }
+        u32x4* to = reinterpret_cast<u32x4*>(cache + lay.value_offset(g_page[0], g, g_pos[0] & (lay.page_size - 1), d));
+        to[0] = lo.u;
+        to[1] = hi.u;
+      } else {
+        for (int j = 0; j < count; ++j)
+          cache[lay.value_offset(g_page[j], g, g_pos[j] & (lay.page_size - 1), d)] = finite_bf16(columns[j][c]);
+      }
+    }
+    return;
+  }
+  id -= value_groups * value_parts;
+  const bool is_q = id < n;
+  const int t = is_q ? id : id - n, pos = positions[t], dk = lay.dk;
+  const int turning = half / 8, per_head = turning + (dk - 2 * half) / 8;        // pieces of a head, those of pairs first
+  const int heads = is_q ? num_heads : lay.kv_heads, total = heads * per_head;
+  const bf16_t* row = is_q ? q + (int64_t)t * ldq : k + (int64_t)t * ldk;
+  const float* bias = is_q ? q_bias : k_bias;
+  const float* weight = is_q ? q_weight : k_weight;
+  float a[R][8], b[R][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int item = r * 256 + tid, h = item / per_head, piece = item - h * per_head;
+    const bool mine = item < total, pairs = mine && piece < turning;
+    const int at = mine ? h * dk + (pairs ? piece * 8 : 2 * half + (piece - turning) * 8) : 0;
+    float part = 0.f;
+    Eight x, y;
+    x.u = *reinterpret_cast<const u32x4*>(row + at);
+    y.u = *reinterpret_cast<const u32x4*>(row + (pairs ? at + half : at));
+    float add_a[8], add_b[8];
+    eight_floats(add_a, bias != nullptr ? bias + at : nullptr, 0.f);
+    eight_floats(add_b, bias != nullptr ? bias + (pairs ? at + half : at) : nullptr, 0.f);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      a[r][i] = bf16_to_float(x.e[i]) + add_a[i];
+      b[r][i] = bf16_to_float(y.e[i]) + add_b[i];
+      part = fmaf(a[r][i], a[r][i], part);
+      if (pairs) part = fmaf(b[r][i], b[r][i], part);
+    }
+    if (!mine) part = 0.f;
+    if constexpr (NORM == 1) sums[item] = part;
+    ss += part;
+  }
+  float inv = 1.0f;
+  if constexpr (NORM == 1) __syncthreads();
+  if constexpr (NORM == 2) inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)(heads * dk) + eps);
+  int page = 0, slot = 0;
+  if (!is_q) {
+    page = block_tables[(int64_t)token_segment[t] * bt_stride + (pos >> lay.page_shift)];
+    slot = pos & (lay.page_size - 1);
+  }
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int item = r * 256 + tid, h = item / per_head, piece = item - h * per_head;
+    if (item >= total) continue;
+    const bool pairs = piece < turning;
+    const int d = pairs ? piece * 8 : 2 * half + (piece - turning) * 8;
+    if constexpr (NORM == 1) {
+      float sum = 0.f;
+      for (int j = 0; j < per_head; ++j) sum += sums[h * per_head + j];
+      inv = 1.0f / sqrtf(sum / (float)dk + eps);
+    }
+    const float* w = weight != nullptr ? weight + (NORM == 2 ? h * dk : 0) + d : nullptr;
+    float wa[8], wb[8];
+    eight_floats(wa, w, 1.0f);
+    Eight x, y;
+    if (pairs) {
+      float c[8], s[8];
+      eight_floats(wb, w != nullptr ? w + half : nullptr, 1.0f);
+      eight_floats(c, cos_t + (int64_t)pos * half + d, 1.0f);
+      eight_floats(s, sin_t + (int64_t)pos * half + d, 0.0f);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float u = a[r][i] * inv * wa[i], z = b[r][i] * inv * wb[i];
+        x.e[i] = float_to_bf16(u * c[i] - z * s[i]);
+        y.e[i] = float_to_bf16(z * c[i] + u * s[i]);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x.e[i] = float_to_bf16(a[r][i] * inv * wa[i]);
+      y.u = x.u;
+    }
+    if (!is_q) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        x.u[i] = finite_bf16x2(x.u[i]);
+        y.u[i] = finite_bf16x2(y.u[i]);
+      }
+    }
+    bf16_t* to = is_q ? q_out + (int64_t)t * ldqo + (int64_t)h * dk + d : cache + lay.key_offset(page, h, slot, d);
+    *reinterpret_cast<u32x4*>(to) = x.u;
+    if (pairs) *reinterpret_cast<u32x4*>(to + half) = y.u;
+  }
+}
+
 // ---------------------------------------------------------------- pooled blocks
 // One wave a (token, key/value head, 64 of the key's and value's dims): a token at the last position of a block of `pool` positions
 // (position % pool == pool - 1) leaves the block's key and value in the pooled blocks' cache layer under
@@ -602,6 +771,29 @@ HFEE_API int hfee_qkv_write(void* q_out, int64_t ldqo, const void* q, int64_t ld
     HFEE_REQUIRE(v != nullptr && cache != nullptr && token_segment != nullptr && block_tables != nullptr,
                  "qkv_write: k, v, the cache and the block tables come together");
     HFEE_REQUIRE(ldk >= (int64_t)kv_heads * dk && ldv >= (int64_t)kv_heads * dv, "qkv_write: k/v rows too short");
+  }
+  // whole pieces of eight dims, everything where 16-byte accesses can reach it: the kernel in pieces
+  const auto aligned = [](const void* p, int to) { return ((uintptr_t)p & (uintptr_t)(to - 1)) == 0; };
+  const int per_head = half / 8 + (dk - 2 * half) / 8;
+  const int most = (num_heads > kv_heads ? num_heads : kv_heads) * per_head;
+  if (dtype == 1 && k != nullptr && dk % 8 == 0 && half % 8 == 0 && dv % 8 == 0 && most <= 256 * kQkvPieces && ldq % 8 == 0 &&
+      ldk % 8 == 0 && ldv % 8 == 0 && ldqo % 8 == 0 && aligned(q, 16) && aligned(k, 16) && aligned(v, 16) && aligned(q_out, 16) &&
+      aligned(cache, 16) && aligned(q_bias, 16) && aligned(k_bias, 16) && aligned(v_bias, 16) && aligned(q_weight, 16) &&
+      aligned(k_weight, 16) && aligned(cos_t, 16) && aligned(sin_t, 16)) {
+    const int groups = (n + 15) / 16, v_parts = (kv_heads * dv + kQkvValueColumns - 1) / kQkvValueColumns;
+    const int64_t blocks = (int64_t)groups * v_parts + 2 * (int64_t)n;
+    HFEE_REQUIRE(blocks <= 0x7fffffff, "qkv_write: too much work for one launch");
+#define PIECES(NORM, R)                                                                                              \
+    qkv_write_pieces_kernel<NORM, R><<<(unsigned)blocks, 256, 0, stream>>>((bf16_t*)q_out, ldqo, (const bf16_t*)q, ldq,\
+        num_heads, (const bf16_t*)k, ldk, (const bf16_t*)v, ldv, q_bias, k_bias, v_bias, q_weight, k_weight, eps, cos_t,\
+        sin_t, half, positions, token_segment, block_tables, bt_stride, (bf16_t*)cache, lay, n, groups, v_parts)
+#define PICK(R)                                                                                                      \
+    if (norm == 0) PIECES(0, R); else if (norm == 1) PIECES(1, R); else PIECES(2, R)
+    if (most <= 256) { PICK(1); } else { PICK(kQkvPieces); }
+#undef PICK
+#undef PIECES
+    HFEE_CHECK_LAUNCH("qkv_write");
+    return 0;
   }
   // a wave a head where a head needs nothing of the others (or the tokens are few), fewer parts where every part
   // has to sum over the whole row

@@ -119,11 +119,13 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkArgs p) {
   constexpr int TILES = Operands::TILES, PITCH = DT * 16 + 4;
   __shared__ float powers[kChunk + 1];
   __shared__ __attribute__((aligned(16))) float St[kColumns * PITCH];      // S transposed: [column][row]
-  const int seg = blockIdx.z, h = blockIdx.y, len = p.segment_lengths[seg];
+  // (heads first: with a multiple of eight heads a head's workgroups, which read the same queries and keys, run on
+  // one of the eight dies)
+  const int seg = blockIdx.z, h = blockIdx.x, len = p.segment_lengths[seg];
   if (len < kLeastTokens) return;
   make_powers(powers, p.decay[h]);
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
-  const int col = blockIdx.x * kColumns + r;
+  const int col = blockIdx.y * kColumns + r;
   const bool live = col < p.V;
   const int row_first = p.segment_rows[seg], kg = h / (p.heads / p.qk_heads);
   const int blocks = (p.V + 3) / 4, R = p.rows_a_lane;
@@ -136,46 +138,45 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkArgs p) {
     const int d0 = (wave + 4 * tile) * 16 + 4 * g;
 #pragma unroll
     for (int i = 0; i < 4; ++i) S[tile][i] = live && d0 + i < p.D ? head_state[place(d0 + i)] : 0.f;
-    if (wave + 4 * tile < DT) *reinterpret_cast<f32x4*>(&St[r * PITCH + d0]) = S[tile];
   }
 
+  // Every load is made, with a place inside the portion and the head for what lies outside of either (a load behind
+  // a condition would be waited for where it stands): what must not count meets a zero where it is used.
+  const int q_step = 4 * g < p.D ? 4 * g : 0;
   auto load = [&](int first, Operands& o) {
     const int L = min(kChunk, len - first);
     const int64_t row0 = row_first + first;
-    const int64_t qrow = row0 + min(wave * 16 + r, L - 1);
-    const float* qp = p.q + qrow * p.ldq + (int64_t)kg * p.D + 4 * g;
+    const float* qb = p.q + row0 * p.ldq + (int64_t)kg * p.D;
+    const float* kb = p.k + row0 * p.ldk + (int64_t)kg * p.D;
+    const float* vb = p.v + row0 * p.ldv + (int64_t)h * p.V;
+    const float* sb = p.scores + ((int64_t)h * p.rows + row0) * kChunk;
+    const int t = min(wave * 16 + r, L - 1), ldq = (int)p.ldq, ldk = (int)p.ldk, ldv = (int)p.ldv;
 #pragma unroll
-    for (int s = 0; s < DT; ++s) {
-      o.q[s] = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (s * 16 + 4 * g < p.D) o.q[s] = *reinterpret_cast<const f32x4*>(qp + s * 16);
-    }
-    const float* sp = p.scores + ((int64_t)h * p.rows + qrow) * kChunk + 4 * g;
+    for (int s = 0; s < DT; ++s) o.q[s] = *reinterpret_cast<const f32x4*>(qb + t * ldq + (s * 16 + 4 * g < p.D ? s * 16 + 4 * g : q_step));
 #pragma unroll
-    for (int s = 0; s < 4; ++s) o.s[s] = *reinterpret_cast<const f32x4*>(sp + s * 16);
+    for (int s = 0; s < 4; ++s) o.s[s] = *reinterpret_cast<const f32x4*>(sb + t * kChunk + s * 16 + 4 * g);
 #pragma unroll
-    for (int s = 0; s < 4; ++s)
+    for (int e = 0; e < 16; ++e) {
+      const int row = min((e >> 2) * 16 + 4 * g + (e & 3), L - 1);
+      o.v[e] = vb[row * ldv + (live ? col : 0)];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int j = s * 16 + 4 * g + i;
-        const int64_t row = row0 + min(j, L - 1);
-        const float x = p.v[row * p.ldv + (int64_t)h * p.V + (live ? col : 0)];
-        o.v[s * 4 + i] = live && j < L ? x : 0.f;
-#pragma unroll
-        for (int tile = 0; tile < TILES; ++tile) {
-          const int d = (wave + 4 * tile) * 16 + r;
-          const float y = p.k[row * p.ldk + (int64_t)kg * p.D + (d < p.D ? d : 0)];
-          o.k[tile][s * 4 + i] = d < p.D ? y : 0.f;
-        }
+      for (int tile = 0; tile < TILES; ++tile) {
+        const int d = (wave + 4 * tile) * 16 + r;
+        o.k[tile][e] = kb[row * ldk + (d < p.D ? d : 0)];
       }
+    }
+  };
+  auto copy_state = [&]() {      // (rows at and beyond D, where the queries hold other numbers, are zeros)
+#pragma unroll
+    for (int tile = 0; tile < TILES; ++tile) {
+      const int d0 = (wave + 4 * tile) * 16 + 4 * g;
+      if (wave + 4 * tile < DT) *reinterpret_cast<f32x4*>(&St[r * PITCH + d0]) = d0 < p.D ? S[tile] : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
   };
 
-  Operands now;
-  load(0, now);
-  __syncthreads();                                        // the powers and the copy of S are there
-  for (int first = 0; first < len; first += kChunk) {
+  auto step = [&](int first, Operands& now, Operands& next) {
     const int L = min(kChunk, len - first);
-    Operands next;
-    if (first + kChunk < len) load(first + kChunk, next);
+    load(first + kChunk < len ? first + kChunk : first, next);
     // o = a^(t+1) q S + P v: the lane ends with tokens wave * 16 + 4 g + i of its column
     f32x4 o0 = {0.f, 0.f, 0.f, 0.f}, o1 = o0;
 #pragma unroll
@@ -203,7 +204,10 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkArgs p) {
     // S <- a^L S + sum_j a^(L-1-j) k_j v_j^T
     const float all = powers[L];
 #pragma unroll
-    for (int e = 0; e < 16; ++e) now.v[e] *= powers[max(L - 1 - ((e >> 2) * 16 + 4 * g + (e & 3)), 0)];
+    for (int e = 0; e < 16; ++e) {
+      const int j = (e >> 2) * 16 + 4 * g + (e & 3);
+      now.v[e] *= j < L ? powers[L - 1 - j] : 0.f;
+    }
 #pragma unroll
     for (int tile = 0; tile < TILES; ++tile) S[tile] = S[tile] * all;
 #pragma unroll
@@ -212,11 +216,17 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkArgs p) {
       for (int tile = 0; tile < TILES; ++tile)
         S[tile] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.k[tile][e], now.v[e], S[tile], 0, 0, 0);
     __syncthreads();                                      // every wave has read the copy of the old S
-#pragma unroll
-    for (int tile = 0; tile < TILES; ++tile)
-      if (wave + 4 * tile < DT) *reinterpret_cast<f32x4*>(&St[r * PITCH + (wave + 4 * tile) * 16 + 4 * g]) = S[tile];
+    copy_state();
     __syncthreads();
-    now = next;
+  };
+  Operands even, odd;      // (by turns: copying one into the other would wait for the loads)
+  load(0, even);
+  copy_state();
+  __syncthreads();                                        // the powers and the copy of S are there
+  for (int first = 0; first < len; first += 2 * kChunk) {
+    step(first, even, odd);
+    if (first + kChunk >= len) break;
+    step(first + kChunk, odd, even);
   }
 #pragma unroll
   for (int tile = 0; tile < TILES; ++tile) {
@@ -256,7 +266,8 @@ HFEE_API int hfee_linear_chunks(float* out, int64_t ldo, float* state, const flo
   const int chunks = (longest + kChunk - 1) / kChunk;
   chunk_scores_kernel<<<dim3(chunks, heads, segments), 256, 0, stream>>>(p);
   HFEE_CHECK_LAUNCH("linear_chunks (scores)");
-  const dim3 grid((vdim + kColumns - 1) / kColumns, heads, segments);
+  HFEE_REQUIRE((vdim + kColumns - 1) / kColumns <= 65535, "linear_chunks: values too wide");
+  const dim3 grid(heads, (vdim + kColumns - 1) / kColumns, segments);
   if (dim <= 32) chunk_walk_kernel<2><<<grid, 256, 0, stream>>>(p);
   else if (dim <= 64) chunk_walk_kernel<4><<<grid, 256, 0, stream>>>(p);
   else if (dim <= 128) chunk_walk_kernel<8><<<grid, 256, 0, stream>>>(p);

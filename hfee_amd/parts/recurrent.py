@@ -56,6 +56,13 @@ from .base import LazyNorm, Mixer, lookup, register_mixer
 from .kv_attention import product, tiles_of
 
 
+def staggered(width: int) -> int:
+    """A row pitch (in float32) of at least `width` for rows that a kernel reads in columns: an odd number of 256-byte
+    pieces, so that the same column of neighbouring rows lies in different memory channels."""
+    pieces = (width + 63) // 64
+    return 64 * (pieces | 1)
+
+
 class _StateMixer(Mixer):
     graph_safe = True
 
@@ -290,7 +297,7 @@ class Retention(_StateMixer):
         total = self.w_in.shape[0]
         proj = ctx.rows("retention.in", (total + 7) // 8 * 8)[:, :total]
         product(ctx, proj, hn, self.w_in, self.w_in_tiles)
-        qkv = ctx.rows("retention.qkv", self.at_g, torch.float32)
+        qkv = ctx.rows("retention.qkv", staggered(self.at_g), torch.float32)[:, :self.at_g]
         pos = self.position
         cos, sin = (pos.cos, pos.sin) if pos else (None, None)
         # q and k as 2 H heads of one row: rotated, the keys' heads then times dim^(-1/2)
@@ -298,7 +305,7 @@ class Retention(_StateMixer):
                         scaled_from=H, factor=D ** -0.5)
         ops.scan_gate(qkv[:, self.at_v:], proj[:, self.at_v:self.at_g], "cast")
         q, k, v = qkv[:, :self.qk_width], qkv[:, self.qk_width:self.at_v], qkv[:, self.at_v:]
-        o = ctx.rows("retention.read", self.v_width, torch.float32)
+        o = ctx.rows("retention.read", staggered(self.v_width), torch.float32)[:, :self.v_width]
         ops.linear_scan(o, self.state, q, k, v, self.decays, None, rows, lengths, slots, H, H, D, V, "decay_add",
                         decay_per_head=True, **self._in_chunks(ctx, H, D))
         gated = ctx.rows("retention.out", self.v_width)
@@ -360,10 +367,10 @@ class LightningAttention(_StateMixer):
         total = self.w_in.shape[0]
         proj = ctx.rows("lightning.in", (total + 7) // 8 * 8)[:, :total]
         product(ctx, proj, hn, self.w_in, self.w_in_tiles)
-        qkv = ctx.rows("lightning.qkv", self.at_g, torch.float32)
+        qkv = ctx.rows("lightning.qkv", staggered(self.at_g), torch.float32)[:, :self.at_g]
         ops.scan_gate(qkv, proj[:, :self.at_g], "silu")
         q, k, v = qkv[:, :self.qk_width], qkv[:, self.qk_width:self.at_v], qkv[:, self.at_v:]
-        o = ctx.rows("lightning.read", self.v_width, torch.float32)
+        o = ctx.rows("lightning.read", staggered(self.v_width), torch.float32)[:, :self.v_width]
         ops.linear_scan(o, self.state, q, k, v, self.decays, None, rows, lengths, slots, H, H, D, V, "decay_add",
                         decay_per_head=True, **self._in_chunks(ctx, H, D))
         gated = ctx.rows("lightning.out", self.v_width)
