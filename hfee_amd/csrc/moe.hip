@@ -15,7 +15,12 @@
 //
 // router_topk: scores of router logits z (float32 [n, experts], plus a bias an expert where one is given); the
 // `top` largest choose a token's experts (the lower number of two equal ones), its pair weights are the chosen
-// scores: sigmoids, or the softmax over all experts, as they are, or the softmax over the chosen ones only.
+// scores: sigmoids, or the softmax over all experts, as they are, or the softmax over the chosen ones only; or the
+// chosen scores divided by their sum and multiplied by a number.  With groups the experts are cut into equal groups of
+// neighbours, and only those of the groups with the largest best scores can be chosen.
+//
+// An expert number at or beyond the number of stacked matrices stands for no matrix: the kernels here leave such a
+// pair alone (grouped_rows.hip adds what it stands for).
 //
 // The experts' matrices are stacked [experts][rows][columns].  Two forms:
 //
@@ -351,15 +356,23 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
 // logit that is not chosen yet (a bit a share in the lane's own registers says which are); the wave's lanes
 // meet over (logit, number), the larger logit and of two equal ones the lower number, and every lane ends
 // with the same answer.  The sigmoid grows with its argument, so the largest scores are the largest logits.
-constexpr int kRouterMostExperts = 64 * 128;
+constexpr int kRouterMostExperts = 64 * 128, kRouterMostGroups = 512;
+
+struct RouterGroups {
+  int count, keep;       // count 0: no groups
+};
 
 // score_kind 0: a score is sigmoid(z); 1: the softmax of z over all experts; 2: the softmax of z over the chosen
 // experts.  bias (float32 [experts] or null) is part of z.  correction (the same; not with kind 2) is added to a
-// score where the experts are chosen and nowhere else: the weights are the scores.
+// score where the experts are chosen and nowhere else: the weights are the scores.  groups: an expert can be chosen
+// where fewer than `keep` groups come before its own (a larger best choice score, or an equal one and a lower number).
+// renormalize (not with kind 2): the weights are the chosen scores / (their sum + 1e-20) * scale.
 __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restrict__ logits, int64_t ld, int n, int experts,
                                                           int top, int* __restrict__ chosen, float* __restrict__ weights,
                                                           int score_kind, const float* __restrict__ correction,
-                                                          const float* __restrict__ bias) {
+                                                          const float* __restrict__ bias, RouterGroups groups,
+                                                          int renormalize, float scale) {
+  extern __shared__ float group_best[];      // [waves][2][groups.count]: a group's best, and whether it is kept
   const int t = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= n) return;
   const float* row = logits + (int64_t)t * ld;
@@ -376,6 +389,26 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
   auto score = [&](int e) { return score_kind == 1 ? expf(z(e) - zmax) * inv_sum : 1.0f / (1.0f + expf(-z(e))); };
   // without a correction the order of the scores is the order of the logits (both scores grow with them)
   auto choice = [&](int e) { return correction != nullptr ? score(e) + correction[e] : z(e); };
+  float* best_of = group_best + (threadIdx.x >> 6) * 2 * groups.count;
+  float* kept = best_of + groups.count;
+  const int each = groups.count > 0 ? experts / groups.count : experts;
+  if (groups.count > 0) {      // (a wave's own part of LDS: what its lanes wrote is there behind the wave's own wait)
+    for (int g = lane; g < groups.count; g += 64) {
+      float best = choice(g * each);
+      for (int e = g * each + 1; e < (g + 1) * each; ++e) best = fmaxf(best, choice(e));
+      best_of[g] = best;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    for (int g = lane; g < groups.count; g += 64) {
+      int before = 0;
+      for (int o = 0; o < groups.count; ++o) before += best_of[o] > best_of[g] || (best_of[o] == best_of[g] && o < g);
+      kept[g] = before < groups.keep ? 1.f : 0.f;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+  }
+  auto open = [&](int e) { return groups.count == 0 || kept[e / each] != 0.f; };
   float first = 0.f, chosen_sum = 0.f;       // (kind 2: the largest logit, and the sum of the chosen ones' exponentials)
   unsigned long long taken[2] = {0ull, 0ull};
   for (int j = 0; j < top; ++j) {
@@ -383,7 +416,7 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
     int at = 0x7fffffff;
     for (int e = lane, i = 0; e < experts; e += 64, ++i) {
       const float v = choice(e);
-      if (!((taken[i >> 6] >> (i & 63)) & 1ull) && (at == 0x7fffffff || v > best)) { best = v; at = e; }
+      if (!((taken[i >> 6] >> (i & 63)) & 1ull) && open(e) && (at == 0x7fffffff || v > best)) { best = v; at = e; }
     }
 #pragma unroll
     for (int off = 32; off >= 1; off >>= 1) {
@@ -400,7 +433,9 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
         chosen_sum += w;
         weights[(int64_t)t * top + j] = w;
       } else {
-        weights[(int64_t)t * top + j] = score(at);
+        const float w = score(at);
+        chosen_sum += w;
+        weights[(int64_t)t * top + j] = w;
       }
     }
   }
@@ -408,24 +443,34 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
     const float inv = 1.0f / chosen_sum;
     for (int j = 0; j < top; ++j) weights[(int64_t)t * top + j] *= inv;
   }
+  if (renormalize && lane == 0) {
+    const float by = scale / (chosen_sum + 1e-20f);
+    for (int j = 0; j < top; ++j) weights[(int64_t)t * top + j] *= by;
+  }
 }
 
 }  // namespace
 
 HFEE_API int hfee_router_topk(const float* logits, int64_t ld, int n, int experts, int top, int* chosen, float* weights,
-                              int score_kind, const float* correction, const float* bias, hipStream_t stream) {
+                              int score_kind, const float* correction, const float* bias, int group_count, int group_keep,
+                              int renormalize, float scale, hipStream_t stream) {
   HFEE_REQUIRE(score_kind >= 0 && score_kind <= 2, "router_topk: the scores are sigmoids (0), a softmax (1) or a softmax over the chosen (2)");
   HFEE_REQUIRE(score_kind != 2 || correction == nullptr, "router_topk: a softmax over the chosen experts takes no correction");
   HFEE_REQUIRE(n >= 0 && experts >= 1 && experts <= kRouterMostExperts && top >= 1 && top <= experts && ld >= experts,
                "router_topk: a token uses 1 to %d experts (of at most %d), not %d", experts, kRouterMostExperts, top);
+  HFEE_REQUIRE(group_count >= 0 && group_count <= kRouterMostGroups && (group_count == 0 || (experts % group_count == 0 &&
+               group_keep >= 1 && group_keep <= group_count && top <= group_keep * (experts / group_count))),
+               "router_topk: %d experts in %d groups of which %d are kept cannot give a token %d", experts, group_count, group_keep, top);
+  HFEE_REQUIRE(!renormalize || score_kind != 2, "router_topk: a softmax over the chosen experts adds up to one already");
   if (n == 0) return 0;
-  router_topk_kernel<<<(n + 3) / 4, 256, 0, stream>>>(logits, ld, n, experts, top, chosen, weights, score_kind, correction, bias);
+  router_topk_kernel<<<(n + 3) / 4, 256, 4 * 2 * group_count * sizeof(float), stream>>>(
+      logits, ld, n, experts, top, chosen, weights, score_kind, correction, bias, RouterGroups{group_count, group_keep}, renormalize, scale);
   HFEE_CHECK_LAUNCH("router_topk");
   return 0;
 }
 
 // The whole feed-forward in its grouped form, bfloat16: x (float32 [n, width]) += the experts' weighted
-// outputs.  order: int32 [n * top]; tiles: int32 [3 * hfee_moe_group_tiles(n, top, experts) + 1]; act:
+// outputs; x null: a pair's output, not weighted, is left in its row of y (whatever top is).  order: int32 [n * top]; tiles: int32 [3 * hfee_moe_group_tiles(n, top, experts) + 1]; act:
 // bfloat16 [n * top, ff]; y: float32 [n * top, width], needed where top > 1.
 HFEE_API int hfee_moe_group_tiles(int n, int top, int experts) {
   return (int)(((int64_t)n * top + kTilePairs - 1) / kTilePairs) + experts;
@@ -440,12 +485,12 @@ HFEE_API int hfee_moe_grouped(float* x, int64_t ldx, const void* h, int64_t ldh,
   const GateNumbers numbers{limit, sharpness};
   HFEE_REQUIRE(n >= 0 && top >= 1 && experts >= 1 && experts <= 8192 && ff >= 1 && width >= 1, "moe_grouped: bad sizes");
   HFEE_REQUIRE(chosen != nullptr || (table != nullptr && token_ids != nullptr), "moe_grouped: the experts of a token, or a table and the ids");
-  HFEE_REQUIRE(width % 32 == 0 && ff % 32 == 0 && ldh % 8 == 0 && ldx >= width && ldh >= width,
+  HFEE_REQUIRE(width % 32 == 0 && ff % 32 == 0 && ldh % 8 == 0 && (x == nullptr || ldx >= width) && ldh >= width,
                "moe_grouped: the width and the experts' size must be multiples of 32");
   HFEE_REQUIRE(w_gate != nullptr || pair_weights == nullptr, "moe_grouped: experts without a gate take their weights on the input");
   HFEE_REQUIRE(((uintptr_t)h | (uintptr_t)w_gate | (uintptr_t)w_up | (uintptr_t)w_down | (uintptr_t)act) % 16 == 0,
                "moe_grouped: operands must be 16-byte aligned");
-  HFEE_REQUIRE(order != nullptr && tiles != nullptr && act != nullptr && (top == 1 || y != nullptr), "moe_grouped: scratch missing");
+  HFEE_REQUIRE(order != nullptr && tiles != nullptr && act != nullptr && ((top == 1 && x != nullptr) || y != nullptr), "moe_grouped: scratch missing");
   HFEE_REQUIRE((int64_t)n * top < (1 << 30), "moe_grouped: too many pairs");
   if (n == 0) return 0;
   const int most = hfee_moe_group_tiles(n, top, experts);
@@ -461,11 +506,12 @@ HFEE_API int hfee_moe_grouped(float* x, int64_t ldx, const void* h, int64_t ldh,
         act, ff, (const bf16_t*)h, ldh, (const bf16_t*)w_up, nullptr, order, tiles, most, top, ff, width, 0, in_weights, 1.0f,
         GATE_SILU, numbers);
   HFEE_CHECK_LAUNCH("moe_group_up");
+  const bool straight = top == 1 && x != nullptr;
   moe_group_tiled_kernel<2><<<dim3(most, (width + kTileRows - 1) / kTileRows), 256, 0, stream>>>(
-      top == 1 ? (void*)x : (void*)y, top == 1 ? ldx : (int64_t)width, (const bf16_t*)act, ff, (const bf16_t*)w_down, nullptr,
-      order, tiles, most, top, width, ff, top == 1 ? 1 : 0, pair_weights, weight, GATE_SILU, numbers);
+      straight ? (void*)x : (void*)y, straight ? ldx : (int64_t)width, (const bf16_t*)act, ff, (const bf16_t*)w_down, nullptr,
+      order, tiles, most, top, width, ff, straight ? 1 : 0, pair_weights, weight, GATE_SILU, numbers);
   HFEE_CHECK_LAUNCH("moe_group_down");
-  if (top > 1) {
+  if (top > 1 && x != nullptr) {
     int parts = (width + 255) / 256;
     if (parts > 64) parts = 64;
     moe_combine_kernel<<<dim3(n, parts), 256, 0, stream>>>(x, ldx, y, pair_weights, weight, top, width);

@@ -69,7 +69,7 @@ _CORE_SIGNATURES = {
     "hfee_linear_chunks_least": [],
     "hfee_rglru_scan": [P, L, I, P, P, L, P, P, L, P, P, L, P, P, P, P, I, I, I, I, P, L, P],
     "hfee_gate_group_norm": [P, L, I, P, L, P, L, P, I, P, L, P, I, I, F, I, P],
-    "hfee_router_topk": [P, L, I, I, I, P, P, I, P, P, P],
+    "hfee_router_topk": [P, L, I, I, I, P, P, I, P, P, I, I, I, F, P],
     "hfee_add_table_rows": [P, I, I, P, I, P, P],
     "hfee_scaled_add": [P, P, F, P, F, L, P],
     "hfee_scaled_add_norm": [P, P, F, P, I, P, F, I, I, P],
@@ -77,6 +77,10 @@ _CORE_SIGNATURES = {
     "hfee_post_norm": [P, P, F, P, F, F, P, F, P, I, P, P, P, I, I, P],
     "hfee_token_shift": [P, I, P, P, P, P, P, P, P, I, I, P],
     "hfee_softcap": [P, F, L, P],
+    "hfee_group_norm": [P, I, P, P, P, F, I, I, I, P],
+    "hfee_pair_norm_add": [P, P, P, P, P, F, F, F, P, I, P, F, I, I, I, P],
+    "hfee_experts_join": [P, P, I, P, P, I, I, P, L, P, P, L, P, I, P, F, I, I, I, P],
+    "hfee_poly_norm": [P, L, P, L, I, P, F, I, I, P],
     "hfee_head_norm_gate": [P, L, P, L, P, L, I, P, I, I, F, I, I, P],
     "hfee_moe_grouped": [P, L, P, L, P, P, P, P, P, P, P, F, I, I, I, I, I, P, P, P, P, P, I, F, F, P],
     "hfee_moe_up": [P, P, L, P, P, I, P, P, P, I, I, I, I, I, P, I, F, F, P],

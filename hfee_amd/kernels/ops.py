@@ -1250,6 +1250,88 @@ def token_shift(out, x, state, shift, token_segment, segment_rows, segment_lengt
                     _ptr(segment_rows), _ptr(segment_lengths), _ptr(segment_slots), n, d, _stream())
 
 
+def _next_norm(next_out, next_weight, next_eps, next_groups, n, d, what):
+    """The arguments of a launch that goes on with the group norm of the rows it made (next_out None: it does not)."""
+    if next_out is None:
+        return None, 0, None, 0.0, 1
+    _gpu(next_out, next_weight)
+    _check(next_out.is_contiguous() and tuple(next_out.shape) == (n, d), f"{what}: next_out [n, d], contiguous")
+    _check(next_weight.dtype == torch.float32 and next_weight.is_contiguous() and next_weight.numel() == d, f"{what}: next_weight float32 [d]")
+    _check(next_groups >= 1 and d % next_groups == 0, f"{what}: {d} values are not {next_groups} equal groups")
+    return _ptr(next_out), _dt(next_out), _ptr(next_weight), float(next_eps), int(next_groups)
+
+
+def group_norm(out, x, weight, eps: float, groups: int, rows=None):
+    """out[r] = x[rows[r] or r] (float32) with each of `groups` equal parts divided by its own sqrt(mean(part^2) + eps),
+    times weight (float32 [d])."""
+    _gpu(out, x, weight, rows)
+    n, d, _ = _rows2d(out, "group_norm out")
+    _check(x.dtype == torch.float32 and x.is_contiguous() and x.dim() == 2 and x.shape[1] == d, "group_norm: contiguous float32 x")
+    if rows is None:
+        _check(x.shape[0] >= n, "group_norm: fewer input rows than output rows")
+    else:
+        _i32(rows, "group_norm rows", n)
+    o, dt, w, e, g = _next_norm(out, weight, eps, groups, n, d, "group_norm")
+    lib.core().call("hfee_group_norm", o, dt, _ptr(x), _ptr(rows), w, e, g, n, d, _stream())
+
+
+def pair_norm_add(x, y, y2, weight, weight2, eps: float, scales=(1.0, 1.0), next_out=None, next_weight=None, next_eps: float = 0.0,
+                  next_groups: int = 1):
+    """x (float32, the residual stream) += scales[0] * norm(y) * weight + scales[1] * norm(y2) * weight2, norm(v) =
+    v / sqrt(mean(v^2) + eps) over the row; with next_out also next_out = `group_norm` of the new x.  y, y2 float32 like
+    x; the weights float32 [d]."""
+    _gpu(x, y, y2, weight, weight2)
+    n, d, _ = _rows2d(x, "pair_norm_add x")
+    for t in (x, y, y2):
+        _check(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (n, d), "pair_norm_add: contiguous float32 rows of one shape")
+    for w in (weight, weight2):
+        _check(w.dtype == torch.float32 and w.is_contiguous() and w.numel() == d, "pair_norm_add: weights float32 [d]")
+    lib.core().call("hfee_pair_norm_add", _ptr(x), _ptr(y), _ptr(y2), _ptr(weight), _ptr(weight2), float(scales[0]), float(scales[1]),
+                    float(eps), *_next_norm(next_out, next_weight, next_eps, next_groups, n, d, "pair_norm_add"), n, d, _stream())
+
+
+def experts_join(x, y, chosen, weights, experts: int, h, shared=None, gate=None, next_out=None, next_weight=None,
+                 next_eps: float = 0.0, next_groups: int = 1):
+    """x[t] (float32, the residual stream) += what a token's experts make of it.  y: float32 [n * top, d], the outputs
+    of the (token, expert) pairs, or [n, d], their weighted sum; chosen int32 [n, top], weights float32 [n, top]:
+    numbers at and beyond `experts` are experts without matrices that hand on their input h [n, d] (times the
+    weight; their rows of y are not looked at).  shared: float32 [n, d], added too, with gate (float32, one number a
+    row, any stride) times sigmoid(gate[t]).  next_out, ...: as in `pair_norm_add`; next_out and h share a dtype."""
+    _gpu(x, y, chosen, weights, h, shared, gate)
+    n, d, _ = _rows2d(x, "experts_join x")
+    nh, wh, ldh = _rows2d(h, "experts_join h")
+    top = chosen.shape[1]
+    _check(x.dtype == torch.float32 and x.is_contiguous() and nh == n and wh == d, "experts_join: contiguous float32 x, h of its shape")
+    _check(y.dtype == torch.float32 and y.is_contiguous() and y.dim() == 2 and y.shape[1] == d and y.shape[0] in (n, n * top),
+           "experts_join: y float32 [n * top, d] or [n, d]")
+    summed = y.shape[0] == n and top > 1
+    _check(chosen.dtype == torch.int32 and chosen.is_contiguous() and tuple(chosen.shape) == (n, top), "experts_join: chosen int32 [n, top]")
+    _check(weights.dtype == torch.float32 and weights.is_contiguous() and tuple(weights.shape) == (n, top), "experts_join: weights float32 [n, top]")
+    if shared is not None:
+        _check(shared.dtype == torch.float32 and shared.is_contiguous() and tuple(shared.shape) == (n, d), "experts_join: shared like x")
+    ldg = 0
+    if gate is not None:
+        _check(shared is not None and gate.dtype == torch.float32 and gate.dim() == 1 and gate.numel() == n, "experts_join: a gate of one number a row")
+        ldg = gate.stride(0) if n > 1 else 1
+    if next_out is not None:
+        _check(next_out.dtype == h.dtype, "experts_join: next_out in h's dtype")
+    nxt = list(_next_norm(next_out, next_weight, next_eps, next_groups, n, d, "experts_join"))
+    nxt[1] = _dt(h)
+    lib.core().call("hfee_experts_join", _ptr(x), _ptr(y), int(summed), _ptr(chosen), _ptr(weights), top, int(experts), _ptr(h), ldh,
+                    _ptr(shared), _ptr(gate), ldg, *nxt, n, d, _stream())
+
+
+def poly_norm(out, z, numbers, eps: float):
+    """out = a N(z) + b N(z^2) + c N(z^3) + e with numbers = (a, b, c, e) (float32 [4] on the device), powers element by
+    element, N(v) = v / sqrt(mean(v^2) + eps) over the row; out and z in the engine's dtype, out may be z."""
+    _gpu(out, z, numbers)
+    n, w, ldz = _rows2d(z, "poly_norm z")
+    no, wo, ldo = _rows2d(out, "poly_norm out")
+    _check(no == n and wo == w and out.dtype == z.dtype, "poly_norm: shapes and dtypes of z and out")
+    _check(numbers.dtype == torch.float32 and numbers.is_contiguous() and numbers.numel() == 4, "poly_norm: numbers float32 [4]")
+    lib.core().call("hfee_poly_norm", _ptr(out), ldo, _ptr(z), ldz, _dt(z), _ptr(numbers), float(eps), n, w, _stream())
+
+
 def softcap(x, cap: float):
     """x (float32, contiguous, in place) = cap * tanh(x / cap)."""
     _gpu(x)
@@ -1747,12 +1829,16 @@ def moe_up(act, h, w_gate, w_up, top: int, chosen=None, table=None, token_ids=No
 ROUTER_SCORES = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}
 
 
-def router_topk(chosen, weights, logits, top: int, score: str = "sigmoid", correction=None, bias=None):
+def router_topk(chosen, weights, logits, top: int, score: str = "sigmoid", correction=None, bias=None, groups=None,
+                renormalize: bool = False, scale: float = 1.0):
     """chosen (int32 [n, top]) = the experts with the `top` largest choice scores of each row of logits
     (float32 [n, experts]; of equal ones the lower number), weights (float32 [n, top]) their scores.  A score
     is sigmoid(logit), or with score "softmax" the softmax over the row; the choice score is the score plus
     correction (float32 [experts]) where one is given, and the weights never hold it.  score "softmax_chosen": the
-    softmax over the chosen logits only.  bias (float32 [experts]) is added to the logits before everything else."""
+    softmax over the chosen logits only.  bias (float32 [experts]) is added to the logits before everything else.  groups
+    (count, keep): the experts are `count` equal groups of neighbours, and only those of the `keep` groups with the largest
+    best choice scores can be chosen.  renormalize: the weights are divided by their sum (+ 1e-20) and multiplied
+    by `scale`."""
     _gpu(chosen, weights, logits, correction, bias)
     n, E, ld = _f32rows(logits, "router_topk logits")
     _check(score in ROUTER_SCORES, f"router_topk: the scores are {sorted(ROUTER_SCORES)}")
@@ -1765,7 +1851,8 @@ def router_topk(chosen, weights, logits, top: int, score: str = "sigmoid", corre
     if bias is not None:
         _check(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == E, "router_topk: bias float32 [experts]")
     lib.core().call("hfee_router_topk", _ptr(logits), ld, n, E, int(top), _ptr(chosen), _ptr(weights), ROUTER_SCORES[score],
-                    _ptr(correction), _ptr(bias), _stream())
+                    _ptr(correction), _ptr(bias), *((int(groups[0]), int(groups[1])) if groups else (0, 0)), int(renormalize),
+                    float(scale), _stream())
 
 
 def moe_down(x, act, w_down, top: int, weight: float = 1.0, pair_weights=None, chosen=None, table=None, token_ids=None,
@@ -1804,10 +1891,11 @@ def moe_grouped(x, h, w_gate, w_up, w_down, top: int, order, tiles, act, y=None,
     order: int32 [n * top]; tiles: int32 [3 * moe_group_tiles(n, top, experts) + 1]; act: bfloat16
     [n * top, ff]; y: float32 [n * top, width] (where top > 1): scratch.  w_gate None: experts without a gate,
     relu(in_weights[t, j] * (w_up[e_j] @ h[t]))^2 in the gate's place (then without pair_weights).  activation,
-    numbers: as in `moe_up`."""
+    numbers: as in `moe_up`.  x None: the pairs' outputs are left in y as they are, row t * top + j, for
+    `experts_join` (experts at and beyond the stacked ones have no rows)."""
     _gpu(x, h, w_gate, w_up, w_down, order, tiles, act, y, pair_weights, chosen, table, token_ids, in_weights)
     n, width, ldh = _rows2d(h, "moe_grouped h")
-    nx, wx, ldx = _f32rows(x, "moe_grouped x")
+    nx, wx, ldx = _f32rows(x, "moe_grouped x") if x is not None else (n, width, 0)
     E, F, W = w_up.shape
     _check(nx == n and wx == width == W and tuple(w_down.shape) == (E, width, F) and w_up.is_contiguous() and w_down.is_contiguous()
            and (w_gate is None or (w_gate.shape == w_up.shape and w_gate.is_contiguous() and w_gate.dtype == torch.bfloat16)),
@@ -1818,7 +1906,7 @@ def moe_grouped(x, h, w_gate, w_up, w_down, top: int, order, tiles, act, y=None,
     _check(act.is_contiguous() and act.numel() >= n * top * F, "moe_grouped: act [n * top, ff]")
     _check(order.dtype == tiles.dtype == torch.int32 and order.is_contiguous() and tiles.is_contiguous()
            and order.numel() >= n * top and tiles.numel() >= 3 * moe_group_tiles(n, top, E) + 1, "moe_grouped: order and tiles")
-    if top > 1:
+    if top > 1 or x is None:
         _check(y is not None and y.dtype == torch.float32 and y.is_contiguous() and y.numel() >= n * top * width,
                "moe_grouped: y float32 [n * top, width]")
     if pair_weights is not None:

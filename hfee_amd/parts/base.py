@@ -223,6 +223,16 @@ class LazyNorm:
         self._tensor = out
         return dict(out=out, weight=form[0], eps=form[1])
 
+    def offer_rows(self) -> dict:
+        """For the part whose last launch holds whole rows of the new x: the arguments (next_out, next_weight, next_eps,
+        next_groups) with which that launch also makes this norm, in groups too; {} if it cannot be made
+        there.  The part that takes the offer has to fill next_out."""
+        form = getattr(self.norm, "grouped_form_f32", lambda: None)()
+        if form is None or self.x.dtype != torch.float32 or self._tensor is not None or self.pending is not None:
+            return {}
+        self._tensor = self.ctx.rows("block.normed", self.x.shape[1])
+        return dict(next_out=self._tensor, next_weight=form[0], next_eps=form[1], next_groups=form[2])
+
     def row_scale(self):
         """For the consuming part: (emitted tensor, `row_scale` arguments) if a producer has
         done the first half, else None."""

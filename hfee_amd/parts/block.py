@@ -1,7 +1,7 @@
 """How a layer's parts are arranged around the residual stream.
 
 "prenorm" is the reference's block (/root/reference/internal/llm/forward.go:79-115):
-x += mixer(norm(x)); x += feed_forward(norm(x)).
+x += mixer(norm(x)); x += feed_forward(norm(x)); a layer may have no feed-forward.
 
 "sandwich" norms a sub-layer's output as well before it adds it:
 x += norm_b(mixer(norm_a(x))); x += norm_d(feed_forward(norm_c(x))), with four norms of their own
@@ -32,6 +32,8 @@ stream in one launch that also makes the next layer's norm (or the head's) where
 """
 from __future__ import annotations
 
+from dataclasses import replace
+
 import torch
 
 from ..config.specs import LayerSpec
@@ -45,21 +47,26 @@ from .kv_attention import product, tiles_of
 class PreNormBlock(Part):
     def __init__(self, spec: LayerSpec, dtype: torch.dtype):
         self.spec, self.dtype = spec, dtype
-        self.mixer_norm = lookup("norm", spec.mixer_norm.kind)(
-            spec.mixer_norm, spec.name_of("mixer_norm", "mixer_norm.") + "weight")
+        self.mixer_norm = self._norm(spec.mixer_norm, "mixer_norm")
         self.mixer = lookup("mixer", spec.mixer.kind)(spec.mixer, spec.name_of("mixer", "mixer."), dtype)
-        self.feed_forward_norm = lookup("norm", spec.feed_forward_norm.kind)(
-            spec.feed_forward_norm, spec.name_of("feed_forward_norm", "feed_forward_norm.") + "weight")
-        self.feed_forward = lookup("feed_forward", spec.feed_forward.kind)(
-            spec.feed_forward, spec.name_of("feed_forward", "feed_forward."), dtype)
+        self.feed_forward_norm = self.feed_forward = None
+        if spec.feed_forward is not None:
+            self.feed_forward_norm = self._norm(spec.feed_forward_norm, "feed_forward_norm")
+            self.feed_forward = lookup("feed_forward", spec.feed_forward.kind)(
+                spec.feed_forward, spec.name_of("feed_forward", "feed_forward."), dtype)
         self.hidden = spec.hidden
+
+    def _norm(self, norm_spec, role):
+        given = dict(self.spec.names).get(role + "_tensor")       # (a checkpoint whose norms are not called "....weight")
+        name = self.spec.prefix + given if given is not None else self.spec.name_of(role, role + ".") + "weight"
+        return lookup("norm", norm_spec.kind)(norm_spec, name)
 
     def parts(self):
         # (each with the parts it is made of itself: a mixer lists a step behind its projections)
         return [q for p in self._own() for q in p.parts()]
 
     def _own(self):
-        return [self.mixer_norm, self.mixer, self.feed_forward_norm, self.feed_forward]
+        return [p for p in (self.mixer_norm, self.mixer, self.feed_forward_norm, self.feed_forward) if p is not None]
 
     # the layer of the paged cache that a run of this block is given belongs to its mixer
     def cache_spec(self):
@@ -69,7 +76,11 @@ class PreNormBlock(Part):
         return getattr(self.mixer, "key_layout", lambda: None)()
 
     def tensor_specs(self):
-        return [s for p in self._own() for s in p.tensor_specs()]
+        specs = [s for p in self._own() for s in p.tensor_specs()]
+        if self.feed_forward is None:       # (a checkpoint may still carry the norm that nothing reads)
+            norm = self._norm(self.spec.feed_forward_norm, "feed_forward_norm")
+            specs += [replace(s, optional=True) for s in norm.tensor_specs()]
+        return specs
 
     def bind(self, tensors):
         for p in self._own():
@@ -86,6 +97,9 @@ class PreNormBlock(Part):
 
     def forward(self, ctx, x, entry, h_in=None, h_next=None):
         h = h_in if h_in is not None else self.begin(ctx, x)
+        if self.feed_forward is None:
+            self._run(self.mixer, ctx, x, h, h_next, entry.cache, entry.writes_cache)
+            return
         h2 = LazyNorm(ctx, self.feed_forward_norm, x, self.feed_forward.second_half_rows)
         self._run(self.mixer, ctx, x, h, h2, entry.cache, entry.writes_cache)
         self._run(self.feed_forward, ctx, x, h2, h_next)
@@ -135,7 +149,7 @@ class SandwichBlock(Part):
             self.feed_forward = lookup("feed_forward", spec.feed_forward.kind)(
                 spec.feed_forward, spec.name_of("feed_forward", "feed_forward."), dtype)
         for n in (self.mixer_post_norm, self.feed_forward_post_norm):
-            if n is not None and getattr(n, "fused_form", None) is None:
+            if n is not None and (getattr(n, "fused_form", None) is None or getattr(n, "groups", 1) != 1):
                 raise ValueError("a sandwich block norms its sub-layers' outputs with y / sqrt(mean(y^2) + eps) * w")
 
     def _own(self):
@@ -283,7 +297,7 @@ class PostNormBlock(Part):
 
         def norm(norm_spec, role):
             made = lookup("norm", norm_spec.kind)(norm_spec, spec.name_of(role, role + ".weight"))
-            if getattr(made, "fused_form_f32", None) is None:
+            if getattr(made, "fused_form_f32", None) is None or getattr(made, "groups", 1) != 1:
                 raise ValueError("a postnorm block norms its sums with v / sqrt(mean(v^2) + eps) * w")
             return made
         self.mixer_norm = norm(spec.mixer_norm, "mixer_norm")

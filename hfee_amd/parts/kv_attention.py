@@ -11,7 +11,9 @@ with those that the first blending layer of the model computed for the same toke
 With `bias` q, k and v each have one, added to their products; with `qk_norm` "head" q and k are divided by
 their root mean square over each head (eps `norm_eps`) and multiplied by a weight of the head's size that all
 heads share, with "row" by that over all heads of the token and a weight of the whole projection's size, in both
-cases before the rotation.  With `chunk` a query sees the positions of its own chunk, position // chunk, with
+cases before the rotation.  The rotation's pairs may be (i, i + half) or, with neither of these, (2i, 2i + 1): a score is a sum over
+the rotated dims, so the rows of W_q's and W_k's rotated dims are put in the order evens, odds when they are bound, and
+the kernels turn pairs (i, i + half) of that order (the cache holds the keys in it).  With `chunk` a query sees the positions of its own chunk, position // chunk, with
 `window` the last `window` positions, itself included; with `keep_first` it also sees the first so many tokens
 of its sequence.  The pages that a window or a chunk has passed go back to the cache manager, except those that
 hold the first tokens.
@@ -207,9 +209,10 @@ class KvAttention(_KvMixer):
         if self.num_heads % self.kv_heads:
             raise ValueError(f"{self.num_heads} heads are not a multiple of {self.kv_heads} kv heads")
         self.position = lookup("position", spec.position.kind)(spec.position) if spec.position else None
-        if self.position is not None and self.position.pairing != 0:
-            raise ValueError("kv_attention rotates pairs (i, i + half)")
         self.prepares = self.has_bias or self.qk_norm is not None       # (more than a rotation stands before the cache)
+        self.pairing = self.position.pairing if self.position is not None else 0
+        if self.prepares and self.pairing != 0:
+            raise ValueError("with a bias or a norm kv_attention rotates pairs (i, i + half)")
         if self.prepares and self.blend is not None:
             raise ValueError("values are blended as they are projected: no bias or norm beside value_blend")
         self.names = self._names(spec, dict(q="q_proj.weight", k="k_proj.weight", v="v_proj.weight", o="o_proj.weight",
@@ -240,7 +243,8 @@ class KvAttention(_KvMixer):
 
     def bind(self, tensors):
         n = self.names
-        self.w_qkv = torch.cat([tensors.pop(n["q"]), tensors.pop(n["k"]), tensors.pop(n["v"])], dim=0).contiguous()
+        self.w_qkv = torch.cat([self._turned(tensors.pop(n["q"])), self._turned(tensors.pop(n["k"])), tensors.pop(n["v"])],
+                               dim=0).contiguous()
         self.w_o = tensors.pop(n["o"]).contiguous()
         self.sinks = None
         if self.sink == "learned":
@@ -254,6 +258,15 @@ class KvAttention(_KvMixer):
         self.blend_weight = t.reshape(1).to(self.dtype).contiguous() if (t is not None and self.blend == "mix") else None
         self.w_qkv_tiles, self.w_o_tiles = tiles_of(self.dtype, self.w_qkv, self.w_o)
 
+    def _turned(self, w):
+        """The rows of a projection [heads * key_dim, hidden] with each head's rotated dims in the order evens, odds
+        where the rotation's pairs are (2i, 2i + 1)."""
+        if self.pairing == 0:
+            return w
+        turn, r = torch.arange(self.dk, device=w.device), self.position.rotary_dim
+        turn = torch.cat([turn[0:r:2], turn[1:r:2], turn[r:]])
+        return w.view(-1, self.dk, w.shape[1])[:, turn].reshape(w.shape)
+
     def cache_spec(self):
         # (a chunk's first position lies at most `chunk` - 1 before any of its queries, as a window's does)
         return CacheNeed("window" if self.reach else "full", (self.kv_heads, self.dk + self.dv), self.reach, layout=_LAYOUT,
@@ -262,7 +275,8 @@ class KvAttention(_KvMixer):
     def key_layout(self):
         pos = self.position
         made = (self.qk_norm, self.norm_eps if self.qk_norm else None, self.has_bias) if self.prepares else ()
-        return (self.kv_heads, self.dk, self.dv, None if pos is None else pos.signature(), *made)
+        turned = (self.pairing,) if self.pairing else ()
+        return (self.kv_heads, self.dk, self.dv, None if pos is None else pos.signature(), *made, *turned)
 
     def forward_into(self, ctx, out, h, cache_layer: int, writes_cache: bool):
         n = ctx.n

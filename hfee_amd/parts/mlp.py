@@ -10,7 +10,9 @@ the same launch).  `forward_into` writes the result as float32 rows instead of a
 "dense_mlp" is the feed-forward without a gate: down(activation(up(h) + b_up)) + b_down, the
 activation one of `ops.ROW_ACTIVATIONS` ("relu2": the square of relu; "xielu": with two learned numbers
 p, q of a tensor, softplus(p) z^2 + z / 2 above zero and (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2 at
-and below it), the biases optional.  It
+and below it; "poly_norm", not of an element alone: with four learned numbers a, b, c, e of a tensor,
+a N(z) + b N(z^2) + c N(z^3) + e with powers element by element and N a token's row divided by its root mean square (eps
+`norm_eps`)), the biases optional.  It
 writes float32 rows (`forward_into`) and leaves the last bias to whoever adds the rows to the
 residual stream (`output_bias`): a block that norms them first folds it into that launch."""
 from __future__ import annotations
@@ -125,9 +127,12 @@ class DenseMLP(FeedForward):
         self.intermediate = spec.get("intermediate")
         self.activation = spec.get("activation", "relu2")
         self.has_bias = bool(spec.get("bias", False))
-        if self.activation not in ops.ROW_ACTIVATIONS:
-            raise ValueError(f"the dense feed-forward has the activations {sorted(ops.ROW_ACTIVATIONS)}, "
+        if self.activation not in (*ops.ROW_ACTIVATIONS, "poly_norm"):
+            raise ValueError(f"the dense feed-forward has the activations {sorted([*ops.ROW_ACTIVATIONS, 'poly_norm'])}, "
                              f"not {self.activation!r}")
+        self.norm_eps = float(spec.get("norm_eps", 1e-6))
+        if self.activation == "poly_norm" and self.has_bias:
+            raise ValueError("poly_norm takes the up product as it is: no biases beside it")
         self.prefix, self.dtype = prefix, dtype
         given = dict(spec.get("names") or ())
         defaults = dict(up="up_proj.weight", up_bias="up_proj.bias", down="down_proj.weight", down_bias="down_proj.bias",
@@ -143,6 +148,8 @@ class DenseMLP(FeedForward):
                       TensorSpec(n["down_bias"], (self.hidden,), role="vector")]
         if self.activation == "xielu":
             specs.append(TensorSpec(n["activation"], (2,), role="vector"))
+        if self.activation == "poly_norm":
+            specs.append(TensorSpec(n["activation"], (4,), role="vector"))
         return specs
 
     def bind(self, tensors):
@@ -154,6 +161,8 @@ class DenseMLP(FeedForward):
         if self.activation == "xielu":      # (two numbers, read once: the kernels take them as arguments)
             p, q = torch.nn.functional.softplus(tensors.pop(n["activation"]).to(torch.float64).cpu()).tolist()
             self.numbers = (p, 0.5 + q)
+        if self.activation == "poly_norm":
+            self.numbers = tensors.pop(n["activation"]).to(torch.float32).contiguous()
         # a second copy in tiles for steps of up to 64 rows, whose products stream the weights
         self.w_up_tiles = self.w_down_tiles = None
         if self.dtype == torch.bfloat16 and self.hidden % 8 == 0 and self.intermediate % 8 == 0:
@@ -167,20 +176,23 @@ class DenseMLP(FeedForward):
         else:
             ops.linear(out, x, weight, **ctx.workspace.split_scratch(n, weight))
 
-    def forward_into(self, ctx, out, h):
-        """out (float32 [n, hidden]) = down(activation(up(h) + b_up)); `output_bias` is not added."""
+    def _activated(self, ctx, h):
         hn = h.tensor() if isinstance(h, LazyNorm) else h
         act = ctx.rows("dense_mlp.act", self.intermediate)
         self._product(ctx, act, hn, self.w_up, self.w_up_tiles)
-        ops.bias_act(act, act, self.up_bias, self.activation, self.numbers)
-        self._product(ctx, out, act, self.w_down, self.w_down_tiles)
+        if self.activation == "poly_norm":
+            ops.poly_norm(act, act, self.numbers, self.norm_eps)
+        else:
+            ops.bias_act(act, act, self.up_bias, self.activation, self.numbers)
+        return act
+
+    def forward_into(self, ctx, out, h):
+        """out (float32 [n, hidden]) = down(activation(up(h) + b_up)); `output_bias` is not added."""
+        self._product(ctx, out, self._activated(ctx, h), self.w_down, self.w_down_tiles)
 
     def forward_add(self, ctx, x, h):
         if self.output_bias is None:        # the down product adds straight into the stream
-            hn = h.tensor() if isinstance(h, LazyNorm) else h
-            act = ctx.rows("dense_mlp.act", self.intermediate)
-            self._product(ctx, act, hn, self.w_up, self.w_up_tiles)
-            ops.bias_act(act, act, self.up_bias, self.activation, self.numbers)
+            act = self._activated(ctx, h)
             n = act.shape[0]
             if self.w_down_tiles is not None and n <= ops.SKINNY_MAX_ROWS:
                 ops.linear_fused(x, act, self.w_down_tiles, "add", **ctx.workspace.product_scratch(n, self.w_down_tiles))

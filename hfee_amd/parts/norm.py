@@ -2,7 +2,8 @@
 the sum in float32, x the float32 residual stream, y in the engine's dtype (with the parameter
 `weight_offset` the stored weight lies around zero and the norm multiplies by offset + w: the sum
 is made once, in float32, when the weight is bound; with the parameter `one_number` the tensor is a
-single number for all coordinates, spread over a float32 row when it is bound); "layernorm": y = (x - mean) / sqrt(variance + eps) * w
+single number for all coordinates, spread over a float32 row when it is bound; with the parameter
+`groups` the row is cut into that many equal parts, each divided by its own root mean square); "layernorm": y = (x - mean) / sqrt(variance + eps) * w
 with the variance as the mean of the squared deviations and no bias; and "none" for a
 place where a model has no norm (the rows as they are, in the engine's dtype)."""
 from __future__ import annotations
@@ -23,6 +24,9 @@ class RMSNorm(Norm):
         self.width, self.eps, self.name = spec.width, spec.eps, name
         self.offset = float(dict(spec.params).get("weight_offset", 0.0))
         self.one_number = bool(dict(spec.params).get("one_number", False))
+        self.groups = int(dict(spec.params).get("groups", 1))
+        if self.groups < 1 or self.width % self.groups:
+            raise ValueError(f"a norm over {self.width} values cannot cut them into {self.groups} equal groups")
         self.weight = None
 
     def tensor_specs(self):
@@ -37,10 +41,18 @@ class RMSNorm(Norm):
             self.weight = (self.weight.to(torch.float32) + self.offset).contiguous()
 
     def fused_form(self):
-        return self.weight, self.eps
+        """(weight, eps) for the launches that fold in a norm over whole rows; None where there are groups."""
+        return (self.weight, self.eps) if self.groups == 1 else None
 
     def fused_form_f32(self):
-        """(weight as float32, eps), for the launches that take their weights in float32 only."""
+        """(weight as float32, eps), for the launches that take their weights in float32 only; None where there are groups."""
+        return self._form_f32() if self.groups == 1 else None
+
+    def grouped_form_f32(self):
+        """(weight as float32, eps, groups), for the launches that norm the rows they make in groups."""
+        return (*self._form_f32(), self.groups)
+
+    def _form_f32(self):
         if self.weight.dtype == torch.float32:
             return self.weight, self.eps
         if getattr(self, "_weight_f32", None) is None:
@@ -48,7 +60,10 @@ class RMSNorm(Norm):
         return self._weight_f32, self.eps
 
     def forward(self, ctx, out, x, rows=None):
-        ops.rmsnorm(out, x, self.weight, self.eps, rows)
+        if self.groups == 1:
+            ops.rmsnorm(out, x, self.weight, self.eps, rows)
+        else:
+            ops.group_norm(out, x, *self.grouped_form_f32(), rows=rows)
 
 
 @register_norm("layernorm")

@@ -6,6 +6,10 @@ the two is a mixer of the registry with its own spec and its own tensors (under 
 mixer's; at most one of the two may ask for one) and either may keep per-request state.  Both write
 float32 rows; a block that norms a sub-layer's result takes the second rows and the two scales into that
 launch (`forward_into` returns them), any other block gets the weighted sum added to the stream.
+
+With `output_norm_eps` each of the two results is first divided by its root mean square over the row and
+multiplied by a weight of its own (tensor names under the roles left_norm and right_norm): the norms, the weighted
+sum, the addition to the stream and the norm that follows are one launch (`ops.pair_norm_add`).
 """
 from __future__ import annotations
 
@@ -13,6 +17,7 @@ import torch
 
 from ..config.specs import MixerSpec
 from ..kernels import ops
+from ..weights.spec import TensorSpec
 from .base import Mixer, lookup, register_mixer
 
 
@@ -35,6 +40,10 @@ class SideBySide(Mixer):
             raise ValueError("at most one mixer of a pair keeps a growing cache")
         self.cached = self.right if self.right.cache_spec() is not None else self.left
         self.second_half_rows = 0
+        self.norm_eps = spec.get("output_norm_eps")           # None: the results as they are
+        self.norm_names = tuple(prefix + given.get(r, d) for r, d in (("left_norm", "left_norm.weight"), ("right_norm", "right_norm.weight")))
+        self.norm_weights = None
+        self.emits_norm = self.norm_eps is not None           # (that launch holds whole rows)
 
     @property
     def graph_safe(self):
@@ -44,11 +53,16 @@ class SideBySide(Mixer):
         return [*self.left.parts(), *self.right.parts()]
 
     def tensor_specs(self):
-        return self.left.tensor_specs() + self.right.tensor_specs()
+        specs = self.left.tensor_specs() + self.right.tensor_specs()
+        if self.norm_eps is not None:
+            specs += [TensorSpec(n, (self.hidden,), role="vector", init=("one_plus_normal",)) for n in self.norm_names]
+        return specs
 
     def bind(self, tensors):
         self.left.bind(tensors)
         self.right.bind(tensors)
+        if self.norm_eps is not None:
+            self.norm_weights = tuple(tensors.pop(n).to(torch.float32).contiguous() for n in self.norm_names)
 
     def cache_spec(self):
         return self.cached.cache_spec()
@@ -56,14 +70,25 @@ class SideBySide(Mixer):
     def key_layout(self):
         return getattr(self.cached, "key_layout", lambda: None)()
 
-    def forward_into(self, ctx, out, h, cache_layer: int, writes_cache: bool):
-        """out = the left mixer's rows; returns the right mixer's rows and the two scales."""
+    def _both(self, ctx, out, h, cache_layer: int, writes_cache: bool):
         self.left.forward_into(ctx, out, h, cache_layer, writes_cache)
         y2 = ctx.rows("side_by_side.second", self.hidden, torch.float32)
         self.right.forward_into(ctx, y2, h, cache_layer, writes_cache)
-        return dict(y2=y2, scales=self.scales)
+        return y2
 
-    def forward_add(self, ctx, x, h, cache_layer: int, writes_cache: bool):
+    def forward_into(self, ctx, out, h, cache_layer: int, writes_cache: bool):
+        """out = the left mixer's rows; returns the right mixer's rows and the two scales.  (With norms behind the two:
+        out = the whole result; returns None.)"""
+        if self.norm_eps is not None:
+            out.zero_()
+            self.forward_add(ctx, out, h, cache_layer, writes_cache)
+            return None
+        return dict(y2=self._both(ctx, out, h, cache_layer, writes_cache), scales=self.scales)
+
+    def forward_add(self, ctx, x, h, cache_layer: int, writes_cache: bool, then=None):
         y = ctx.rows("mixer.rows_out", self.hidden, torch.float32)
-        second = self.forward_into(ctx, y, h, cache_layer, writes_cache)
-        ops.scaled_add(x, y, self.scales[0], second["y2"], self.scales[1])
+        y2 = self._both(ctx, y, h, cache_layer, writes_cache)
+        if self.norm_eps is None:
+            ops.scaled_add(x, y, self.scales[0], y2, self.scales[1])
+            return
+        ops.pair_norm_add(x, y, y2, *self.norm_weights, self.norm_eps, self.scales, **(then.offer_rows() if then is not None else {}))

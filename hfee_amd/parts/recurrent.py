@@ -13,7 +13,8 @@ become unit vectors per head, x / sqrt(sum(x^2) + unit_eps), q also times dim^(-
 b = sigmoid(W_b h) a head; a = exp(-exp(A_h) softplus(W_a2 W_a1 h + dt_bias)) a head and key channel.
 Per token S <- diag(a) S; u = b (v - S^T k); S <- S + k u^T; o = S^T q.  Each head's o is divided by
 its root mean square (eps `norm_eps`), times a weight shared by the heads, times
-sigmoid(W_g2 W_g1 h); then the output product.
+sigmoid(W_g2 W_g1 h); then the output product.  Without `decay_rank` there is one decay a head, a =
+exp(-exp(A_h) softplus(W_a h + dt_bias)); without `gate_rank` the gate is silu(W_g h).
 
 "gla": q = W_q h dim^(-1/2), k, v; a = sigmoid(W_a2 W_a1 h + bias)^(1/tau);
 S <- diag(a) S + k v^T; o = S^T q; each head's o normed as above with a weight shared by the heads,
@@ -88,6 +89,9 @@ class _StateMixer(Mixer):
 
 @register_mixer("gated_delta")
 class GatedDelta(_StateMixer):
+    """Tensor names by role: q, k, v, b, o (matrices), q_conv, k_conv, v_conv ([channels, taps]), a_log ([heads]), norm
+    ([vdim]), a_down, a_up and dt_bias ([heads * dim]) or a and dt_bias ([heads]), g_down and g_up or g."""
+
     def __init__(self, spec: MixerSpec, prefix: str, dtype: torch.dtype):
         self.prefix, self.dtype = prefix, dtype
         self.hidden = spec.get("hidden")
@@ -105,7 +109,9 @@ class GatedDelta(_StateMixer):
         self.names = self._names(spec, dict(
             q="q_proj.weight", k="k_proj.weight", v="v_proj.weight", q_conv="q_conv.weight", k_conv="k_conv.weight",
             v_conv="v_conv.weight", b="b_proj.weight", a_log="A_log", norm="norm.weight", a_down="a_down.weight",
-            a_up="a_up.weight", dt_bias="dt_bias", g_down="g_down.weight", g_up="g_up.weight", o="o_proj.weight"))
+            a_up="a_up.weight", a="a_proj.weight", dt_bias="dt_bias", g_down="g_down.weight", g_up="g_up.weight",
+            g="g_proj.weight", o="o_proj.weight"))
+        self.decay_per_head, self.gate_activation = self.decay_rank is None, "silu" if self.gate_rank is None else "sigmoid"
         self.qk_width, self.v_width = self.qk_heads * self.dim, self.heads * self.vdim
         self.channels = 2 * self.qk_width + self.v_width
 
@@ -116,26 +122,45 @@ class GatedDelta(_StateMixer):
                  TensorSpec(n["v"], (self.v_width, self.hidden)), TensorSpec(n["v_conv"], (self.v_width, self.taps), role="vector"),
                  TensorSpec(n["b"], (H, self.hidden)), TensorSpec(n["a_log"], (H,), role="vector"),
                  TensorSpec(n["norm"], (self.vdim,), role="vector", init=("one_plus_normal",)),
-                 TensorSpec(n["a_down"], (self.decay_rank, self.hidden)), TensorSpec(n["a_up"], (H * D, self.decay_rank)),
-                 TensorSpec(n["dt_bias"], (H * D,), role="vector"),
-                 TensorSpec(n["g_down"], (self.gate_rank, self.hidden)), TensorSpec(n["g_up"], (self.v_width, self.gate_rank)),
+                 TensorSpec(n["dt_bias"], (H if self.decay_per_head else H * D,), role="vector"),
                  TensorSpec(n["o"], (self.hidden, self.v_width))]
+        if self.decay_per_head:
+            specs.append(TensorSpec(n["a"], (H, self.hidden)))
+        else:
+            specs += [TensorSpec(n["a_down"], (self.decay_rank, self.hidden)), TensorSpec(n["a_up"], (H * D, self.decay_rank))]
+        if self.gate_rank is None:
+            specs.append(TensorSpec(n["g"], (self.v_width, self.hidden)))
+        else:
+            specs += [TensorSpec(n["g_down"], (self.gate_rank, self.hidden)), TensorSpec(n["g_up"], (self.v_width, self.gate_rank))]
         return specs
 
     def bind(self, tensors):
         n = self.names
         f32 = lambda name: tensors.pop(name).to(torch.float32).contiguous()      # noqa: E731
-        # one product for everything that reads the layer's input: [q | k | v | a_down | g_down | b]
-        self.w_in = torch.cat([tensors.pop(n[r]) for r in ("q", "k", "v", "a_down", "g_down", "b")], dim=0).contiguous()
-        self.at_a = self.channels
-        self.at_g = self.at_a + self.decay_rank
-        self.at_b = self.at_g + self.gate_rank
+        # one product for everything that reads the layer's input: [q | k | v | gate or its first half | decay or its
+        # first half | b]  (with both halves: the decay's first half first)
+        parts = [("a" if self.decay_per_head else "a_down", self.heads if self.decay_per_head else self.decay_rank),
+                 ("g" if self.gate_rank is None else "g_down", self.v_width if self.gate_rank is None else self.gate_rank)]
+        if self.gate_rank is None:
+            parts.reverse()
+        self.w_in = torch.cat([tensors.pop(n[r]) for r in ("q", "k", "v", parts[0][0], parts[1][0], "b")], dim=0)
+        # (filled up with rows of zeros to a multiple of 8, so that blocks of columns stay aligned and the rows fill tiles)
+        self.w_in = F.pad(self.w_in, (0, 0, 0, -self.w_in.shape[0] % 8)).contiguous()
+        second = self.channels + parts[0][1]
+        self.at_b = second + parts[1][1]
+        self.a_columns = slice(self.channels, second) if self.gate_rank is not None else slice(second, self.at_b)
+        self.g_columns = slice(second, self.at_b) if self.gate_rank is not None else slice(self.channels, second)
         self.conv_taps = torch.cat([f32(n["q_conv"]), f32(n["k_conv"]), f32(n["v_conv"])], dim=0).contiguous()
         self.a_log, self.dt_bias, self.norm_weight = f32(n["a_log"]), f32(n["dt_bias"]), f32(n["norm"])
-        self.w_a_up, self.w_g_up = tensors.pop(n["a_up"]).contiguous(), tensors.pop(n["g_up"]).contiguous()
         self.w_o = tensors.pop(n["o"]).contiguous()
-        self.w_in_tiles, self.w_o_tiles = tiles_of(self.dtype, self.w_in, self.w_o)
-        self.w_a_up_tiles, self.w_g_up_tiles = tiles_of(self.dtype, self.w_a_up, self.w_g_up)
+        self.w_in_tiles, = tiles_of(self.dtype, self.w_in)
+        self.w_o_tiles, = tiles_of(self.dtype, self.w_o)
+        if not self.decay_per_head:
+            self.w_a_up = tensors.pop(n["a_up"]).contiguous()
+            self.w_a_up_tiles, = tiles_of(self.dtype, self.w_a_up)
+        if self.gate_rank is not None:
+            self.w_g_up = tensors.pop(n["g_up"]).contiguous()
+            self.w_g_up_tiles, = tiles_of(self.dtype, self.w_g_up)
 
     def state_specs(self):
         return [(self.prefix + "state", (self.heads, *ops.scan_state_shape(self.dim, self.vdim)), torch.float32),
@@ -146,11 +171,16 @@ class GatedDelta(_StateMixer):
         self.conv_state = info.storage.states[self.prefix + "conv_state"]
 
     def forward_add(self, ctx, x, h, cache_layer: int, writes_cache: bool):
+        self._run(ctx, x, h, add=True)
+
+    def forward_into(self, ctx, out, h, cache_layer: int, writes_cache: bool):
+        self._run(ctx, out, h, add=False)
+
+    def _run(self, ctx, x, h, add: bool):
         hn = h.tensor() if isinstance(h, LazyNorm) else h
         H, G, D, V = self.heads, self.qk_heads, self.dim, self.vdim
         rows, lengths, slots = self._segments(ctx)
-        total = self.w_in.shape[0]       # (rows of a multiple of 8 elements, so that blocks of columns stay aligned)
-        proj = ctx.rows("gated_delta.in", (total + 7) // 8 * 8)[:, :total]
+        proj = ctx.rows("gated_delta.in", self.w_in.shape[0])
         product(ctx, proj, hn, self.w_in, self.w_in_tiles)
         raw = proj[:, :self.channels]
         y = ctx.rows("gated_delta.conv", self.channels, torch.float32)
@@ -159,19 +189,25 @@ class GatedDelta(_StateMixer):
         q, k, v = y[:, :self.qk_width], y[:, self.qk_width:2 * self.qk_width], y[:, 2 * self.qk_width:]
         ops.unit_heads(q, G, D, self.unit_eps, D ** -0.5)
         ops.unit_heads(k, G, D, self.unit_eps, 1.0)
-        step = ctx.rows("gated_delta.step", H * D)
-        product(ctx, step, proj[:, self.at_a:self.at_g], self.w_a_up, self.w_a_up_tiles)
-        decay = ctx.rows("gated_delta.decay", H * D, torch.float32)
-        ops.scan_gate(decay, step, "step_decay", bias=self.dt_bias, per_head=self.a_log, head_width=D)
+        per_decay = 1 if self.decay_per_head else D
+        step = proj[:, self.a_columns]
+        if not self.decay_per_head:
+            step = ctx.rows("gated_delta.step", H * D)
+            product(ctx, step, proj[:, self.a_columns], self.w_a_up, self.w_a_up_tiles)
+        decay = ctx.rows("gated_delta.decay", H * per_decay, torch.float32)
+        ops.scan_gate(decay, step, "step_decay", bias=self.dt_bias, per_head=self.a_log, head_width=per_decay)
         beta = ctx.rows("gated_delta.beta", H, torch.float32)
         ops.scan_gate(beta, proj[:, self.at_b:self.at_b + H], "sigmoid")
         o = ctx.rows("gated_delta.read", self.v_width, torch.float32)
-        ops.linear_scan(o, self.state, q, k, v, decay, beta, rows, lengths, slots, H, G, D, V, "delta")
-        gate = ctx.rows("gated_delta.gate", self.v_width)
-        product(ctx, gate, proj[:, self.at_g:self.at_b], self.w_g_up, self.w_g_up_tiles)
+        ops.linear_scan(o, self.state, q, k, v, decay, beta, rows, lengths, slots, H, G, D, V, "delta",
+                        decay_per_head=self.decay_per_head)
+        gate = proj[:, self.g_columns]
+        if self.gate_rank is not None:
+            gate = ctx.rows("gated_delta.gate", self.v_width)
+            product(ctx, gate, proj[:, self.g_columns], self.w_g_up, self.w_g_up_tiles)
         gated = ctx.rows("gated_delta.out", self.v_width)
-        ops.head_norm_gate(gated, o, gate, self.norm_weight, H, V, self.norm_eps, "sigmoid")
-        product(ctx, x, gated, self.w_o, self.w_o_tiles, add=True)
+        ops.head_norm_gate(gated, o, gate, self.norm_weight, H, V, self.norm_eps, self.gate_activation)
+        product(ctx, x, gated, self.w_o, self.w_o_tiles, add=add)
 
 
 @register_mixer("gla")

@@ -12,7 +12,9 @@ use (/root/reference/internal/llm/forward.go:186).  Here a table [positions, dim
 of cos and sin is made once from those float64 angles and rounded to float32, so
 large positions lose nothing to a float32 angle.
 
-A second stretching rule, "yarn": (kind, factor, original context, fast, slow).  With
+The simplest stretching rule, "linear": (kind, factor): every frequency is divided by `factor`.
+
+A third rule, "yarn": (kind, factor, original context, fast, slow).  With
 turn(t) = dim * ln(original / (2 pi t)) / (2 ln theta), the dimension whose wave makes t turns over
 the original context, the dimensions up to lo = max(floor(turn(fast)), 0) keep their frequency,
 those from hi = min(ceil(turn(slow)), dim - 1) on are divided by `factor`, and between them the
@@ -37,6 +39,8 @@ def rope_frequencies(rotary_dim: int, theta: float, scaling=None) -> np.ndarray:
     inv = np.array([1.0 / math.pow(theta, (2 * i) / rotary_dim) for i in range(half)], dtype=np.float64)
     if scaling is None:
         return inv
+    if scaling[0] == "linear":
+        return inv / float(scaling[1])
     if scaling[0] == "yarn":
         _, factor, original, fast, slow = scaling
 
