@@ -95,6 +95,14 @@ SAPOSUN_SIZES = {
 # sixteen routed experts, two a token, and one of the same size that every token uses.
 MEDULORN_SIZES = SAPOSUN_SIZES
 
+# The Miberax design at the same two layer sizes, beside Medulorn (the closest of the other designs: attention over
+# chunks, a pair of attention and a recurrence, clipped experts beside one for every token): every layer is a pair of
+# attention over chunks of 1,536 keys (heads and head size of the Llama layer of that width) and the gated delta rule
+# (Sabezen's heads); two layers of three have sixteen routed experts and four that hand on their input, in four groups
+# of which two are kept, two a token, and one of the same size that every token uses behind a gate, the third has
+# the dense feed-forward of Sabezen's size.
+MIBERAX_SIZES = SABEZEN_SIZES
+
 CONTEXT = 8192
 PROMPT = 1024
 PREFILL = 2048
@@ -166,6 +174,13 @@ def parse(argv=None):
                     help="with --medulorn: only this layer size")
     ap.add_argument("--medulorn-design", choices=["both", "medulorn", "saposun"], default="both",
                     help="with --medulorn: only one of the two designs (for profiling)")
+    ap.add_argument("--miberax", action="store_true",
+                    help="the Miberax design beside Medulorn at equal layer sizes instead of the serving benchmark: its own "
+                    "JSON line, prefill of 2,048 tokens and decode at --batch")
+    ap.add_argument("--miberax-size", choices=sorted(MIBERAX_SIZES), default=None,
+                    help="with --miberax: only this layer size")
+    ap.add_argument("--miberax-design", choices=["both", "miberax", "medulorn"], default="both",
+                    help="with --miberax: only one of the two designs (for profiling)")
     ap.add_argument("--no-extra-points", action="store_true",
                     help="skip the other shapes and the longer context that the default run adds under `points`")
     return ap.parse_args(argv)
@@ -323,6 +338,21 @@ def medulorn_config(size: dict, layers: int, vocab: int = 32000) -> dict:
             "layers": [dict((att, pair)[i % 2], mlp=moe) for i in range(layers)]}
 
 
+def miberax_config(size: dict, layers: int, vocab: int = 32000) -> dict:
+    d, H, G, hd = size["width"], size["heads"], size["kv_heads"], size["dim"]
+    heads = d // 256
+    left = {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": 1536},
+            "rot": {"base": 500000.0, "dims": hd, "scaling": {"factor": 4.0}}}
+    right = {"heads": heads, "kv_heads": max(1, heads // 2), "dim": 128, "vdim": 256, "conv": 4}
+    moe = {"kind": "moe", "expert": {"ff": size["expert_ff"], "limit": 7.0},
+           "router": {"experts": 16, "identity": 4, "groups": {"count": 4, "keep": 2}, "top": 2, "scale": 1.0},
+           "shared": {"ff": size["expert_ff"], "limit": 7.0}}
+    dense = {"kind": "dense", "ff": size["ff"]}
+    return {"architecture": "Miberax", "vocab": vocab, "width": d, "norm": {"eps": 1e-5, "groups": 4}, "max_positions": 4096,
+            "layers": [{"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": (moe, moe, dense)[i % 3]}
+                       for i in range(layers)]}
+
+
 def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
     """Prefill of 2,048 tokens and decode at `batch` requests of 1,024-token prompts for any
     registered architecture: times, and the fractions of the HBM and matrix peaks by the bytes a
@@ -347,12 +377,15 @@ def design_point(cj: dict, batch: int, steps: int, warmup: int) -> dict:
             if f.get("shared") is not None:      # (the expert that every token uses, before the others' prefix)
                 shared = ls.name_of("feed_forward", "") + dict(f.get("names")).get("shared")
                 used[shared] = read[shared] = 1.0
-            used[ls.name_of("feed_forward", "")] = f.get("top") / f.get("experts")
-            read[ls.name_of("feed_forward", "")] = min(1.0, batch * f.get("top") / f.get("experts"))
+            chosen = f.get("top") / (f.get("experts") + (f.get("identity") or 0))
+            used[ls.name_of("feed_forward", "")] = chosen
+            read[ls.name_of("feed_forward", "")] = min(1.0, batch * chosen)
 
     def share(t, table):
         return next((v for k, v in table.items() if t.name.startswith(k)), 1.0)
     weight_bytes = 2 * sum(t.shape[0] * t.shape[1] * share(t, read) for t in matrices)
+    if spec.head_name is None:      # (the head reads the embedding's table)
+        weight_bytes += 2 * spec.vocab * spec.hidden
     layer_flops_a_token = 2 * sum(t.shape[0] * t.shape[1] * share(t, used) for t in matrices)
     attention_dims = 0          # (key size + value size) x heads, summed over the layers, as the kernels see them
     chunked_flops = 0.0         # attention over chunks: the keys that a prompt of PREFILL tokens sees
@@ -521,6 +554,23 @@ def medulorn_compare(args) -> dict:
             "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16", "layers": layers, "points": points}
 
 
+def miberax_compare(args) -> dict:
+    import hfee_amd  # noqa: F401
+    layers = args.layers or 6
+    points = {}
+    for name, size in MIBERAX_SIZES.items():
+        if args.miberax_size not in (None, name):
+            continue
+        for design, cj in (("miberax", miberax_config(size, layers)), ("medulorn", medulorn_config(MEDULORN_SIZES[name], layers))):
+            if args.miberax_design not in ("both", design):
+                continue
+            print(f"[bench] {design} {name}, {layers} layers", file=sys.stderr, flush=True)
+            points[f"{design}_{name}"] = design_point(cj, args.batch, min(args.steps, 32), min(args.warmup, 4))
+    return {"metric": "Miberax beside Medulorn at equal layer sizes: prefill of 2,048 tokens, decode at batch %d and "
+                      "1,024-token prompts (bf16, random weights)" % args.batch,
+            "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16", "layers": layers, "points": points}
+
+
 def sabezen_compare(args) -> dict:
     import hfee_amd  # noqa: F401
     layers = args.layers or 6
@@ -544,6 +594,9 @@ def main(argv=None) -> int:
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")
         return 2
+    if args.miberax:
+        print(json.dumps(miberax_compare(args)), flush=True)
+        return 0
     if args.medulorn:
         print(json.dumps(medulorn_compare(args)), flush=True)
         return 0

@@ -347,8 +347,8 @@ struct RowShape {
   int held, threads;
 };
 RowShape row_shape(bool fits, int d) {
-  if (!fits || d % 4 != 0 || d > 16384) return {0, 256};
-  const int fours = d / 4, held = fours <= 1024 ? 1 : fours <= 2048 ? 2 : 4;
+  if (!fits || d % 4 != 0 || d > 32768) return {0, 256};
+  const int fours = d / 4, held = fours <= 1024 ? 1 : fours <= 2048 ? 2 : fours <= 4096 ? 4 : 8;
   int threads = ((fours + held - 1) / held + 63) / 64 * 64;
   return {held, threads > 1024 ? 1024 : threads};
 }
@@ -373,7 +373,8 @@ int check_next(const NextNorm& to, int dtype, int d, const char* what) {
     if ((shape).held == 0) LAUNCH(T, 0);                                                                             \
     else if ((shape).held == 1) LAUNCH(T, 1);                                                                        \
     else if ((shape).held == 2) LAUNCH(T, 2);                                                                        \
-    else LAUNCH(T, 4);                                                                                               \
+    else if ((shape).held == 4) LAUNCH(T, 4);                                                                        \
+    else LAUNCH(T, 8);                                                                                               \
   } while (0)
 
 // out: [n, d] in dtype (0 float32, 1 bfloat16), contiguous; x: float32, contiguous rows; w: float32 [d].

@@ -449,6 +449,67 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const float* __restric
   }
 }
 
+// The same for up to 64 experts, one a lane: a lane keeps its expert's score and choice score in registers.
+__global__ __launch_bounds__(256) void router_topk_few_kernel(const float* __restrict__ logits, int64_t ld, int n, int experts,
+                                                              int top, int* __restrict__ chosen, float* __restrict__ weights,
+                                                              int score_kind, const float* __restrict__ correction,
+                                                              const float* __restrict__ bias, RouterGroups groups,
+                                                              int renormalize, float scale) {
+  const int t = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (t >= n) return;
+  const bool mine = lane < experts;
+  const int e = mine ? lane : 0;
+  float z = logits[(int64_t)t * ld + e];
+  if (bias != nullptr) z += bias[e];
+  const float shift = correction != nullptr ? correction[e] : 0.f;
+  float score = z;                                       // (kind 2: the exponential comes when the largest is known)
+  if (score_kind == 0) score = 1.0f / (1.0f + expf(-z));
+  if (score_kind == 1) {
+    const float zmax = wave_max(mine ? z : -INFINITY);
+    const float w = expf(z - zmax);
+    score = w * (1.0f / wave_sum(mine ? w : 0.f));
+  }
+  // without a correction the order of the scores is the order of the logits (both scores grow with them)
+  const float choice = correction != nullptr ? score + shift : z;
+  bool open = mine;
+  if (groups.count > 0) {
+    const int each = experts / groups.count, first = e / each * each;
+    float best = -INFINITY;
+    for (int i = 0; i < each; ++i) best = fmaxf(best, __shfl(choice, first + i, 64));
+    int before = 0;
+    for (int o = 0; o < experts; o += each) {
+      const float other = __shfl(best, o, 64);
+      before += other > best || (other == best && o < first);
+    }
+    open = mine && before < groups.keep;
+  }
+  float first_choice = 0.f, sum = 0.f, kept = 0.f;       // kept: lane j's weight of the j-th chosen
+  int kept_at = 0;
+  for (int j = 0; j < top; ++j) {
+    float best = choice;
+    int at = open ? lane : 0x7fffffff;
+#pragma unroll
+    for (int off = 32; off >= 1; off >>= 1) {
+      const float ob = __shfl_xor(best, off, 64);
+      const int oa = __shfl_xor(at, off, 64);
+      if (oa != 0x7fffffff && (at == 0x7fffffff || ob > best || (ob == best && oa < at))) { best = ob; at = oa; }
+    }
+    if (j == 0) first_choice = best;
+    const float w = score_kind == 2 ? expf(best - first_choice) : __shfl(score, at & 63, 64);
+    sum += w;
+    if (at == lane) open = false;
+    if (j == lane) {
+      kept = w;
+      kept_at = at;
+    }
+  }
+  if (lane >= top) return;                               // (top is at most the number of experts)
+  if (score_kind == 2) kept *= 1.0f / sum;
+  if (renormalize) kept *= scale / (sum + 1e-20f);
+  chosen[(int64_t)t * top + lane] = kept_at;
+  weights[(int64_t)t * top + lane] = kept;
+}
+
 }  // namespace
 
 HFEE_API int hfee_router_topk(const float* logits, int64_t ld, int n, int experts, int top, int* chosen, float* weights,
@@ -463,6 +524,12 @@ HFEE_API int hfee_router_topk(const float* logits, int64_t ld, int n, int expert
                "router_topk: %d experts in %d groups of which %d are kept cannot give a token %d", experts, group_count, group_keep, top);
   HFEE_REQUIRE(!renormalize || score_kind != 2, "router_topk: a softmax over the chosen experts adds up to one already");
   if (n == 0) return 0;
+  if (experts <= 64) {
+    router_topk_few_kernel<<<(n + 3) / 4, 256, 0, stream>>>(logits, ld, n, experts, top, chosen, weights, score_kind, correction,
+                                                            bias, RouterGroups{group_count, group_keep}, renormalize, scale);
+    HFEE_CHECK_LAUNCH("router_topk");
+    return 0;
+  }
   router_topk_kernel<<<(n + 3) / 4, 256, 4 * 2 * group_count * sizeof(float), stream>>>(
       logits, ld, n, experts, top, chosen, weights, score_kind, correction, bias, RouterGroups{group_count, group_keep}, renormalize, scale);
   HFEE_CHECK_LAUNCH("router_topk");

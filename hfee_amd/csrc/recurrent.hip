@@ -370,6 +370,47 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(T* __restrict__ out
   }
 }
 
+// The same for heads of whole groups of four, up to 1,024 values: 2^k neighbouring lanes a (token, head), each with up to
+// four fours of it in registers between the sum and the product.
+template <typename T>
+__global__ __launch_bounds__(256) void head_norm_gate_fours_kernel(T* __restrict__ out, int64_t ldo, const float* __restrict__ o,
+                                                                   int64_t ldi, const T* __restrict__ gate, int64_t ldg,
+                                                                   const float* __restrict__ weight, int heads, int V,
+                                                                   float eps, int act, int64_t items, int lanes) {
+  const int64_t item = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) / lanes;
+  const int part = threadIdx.x & (lanes - 1);
+  const bool live = item < items;
+  const int64_t t = (live ? item : 0) / heads, h = (live ? item : 0) % heads;
+  const float* p = o + t * ldi + h * V;
+  const T* g = gate + t * ldg + h * V;
+  float v[4][4], z[4][4], w[4][4], ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const int d = (k * lanes + part) * 4;
+    if (k > 0 && k * lanes * 4 >= V) break;
+    const int dd = d < V ? d : 0;
+    load4<float>(v[k], p + dd);
+    load4<T>(z[k], g + dd);
+    load4<float>(w[k], weight + dd);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) ss = d < V ? fmaf(v[k][i], v[k][i], ss) : ss;
+  }
+  for (int off = lanes >> 1; off > 0; off >>= 1) ss += __shfl_xor(ss, off, kWave);
+  const float inv = 1.0f / sqrtf(ss / (float)V + eps);
+  if (!live) return;
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const int d = (k * lanes + part) * 4;
+    if (d >= V) break;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float sig = 1.0f / (1.0f + expf(-z[k][i]));
+      v[k][i] = v[k][i] * inv * w[k][i] * (act == 0 ? sig : z[k][i] * sig);
+    }
+    store4<T>(out + t * ldo + h * V + d, v[k]);
+  }
+}
+
 // The same with a workgroup a (token, head), for heads of many values (all heads of a token normed together as one).
 template <typename T>
 __global__ __launch_bounds__(1024) void wide_head_norm_gate_kernel(T* __restrict__ out, int64_t ldo, const float* __restrict__ o,
@@ -745,6 +786,20 @@ HFEE_API int hfee_head_norm_gate(void* out, int64_t ldo, const float* o, int64_t
                                                                                  ldg, weight, heads, vdim, eps, act);
     else
       return fail("head_norm_gate: unknown dtype %d", dtype);
+    HFEE_CHECK_LAUNCH("head_norm_gate");
+    return 0;
+  }
+  if (vdim % 4 == 0 && ldo % 4 == 0 && ldi % 4 == 0 && ldg % 4 == 0 && (dtype == 0 || dtype == 1) &&
+      (((uintptr_t)out | (uintptr_t)o | (uintptr_t)gate | (uintptr_t)weight) & 15) == 0) {
+    int lanes = 1;
+    while (lanes < 64 && lanes * 4 < vdim) lanes *= 2;
+    const unsigned groups = (unsigned)((items * lanes + 255) / 256);
+    if (dtype == 0)
+      head_norm_gate_fours_kernel<float><<<groups, 256, 0, stream>>>((float*)out, ldo, o, ldi, (const float*)gate, ldg, weight,
+                                                                     heads, vdim, eps, act, items, lanes);
+    else
+      head_norm_gate_fours_kernel<bf16_t><<<groups, 256, 0, stream>>>((bf16_t*)out, ldo, o, ldi, (const bf16_t*)gate, ldg, weight,
+                                                                      heads, vdim, eps, act, items, lanes);
     HFEE_CHECK_LAUNCH("head_norm_gate");
     return 0;
   }

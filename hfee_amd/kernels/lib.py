@@ -77,6 +77,10 @@ _CORE_SIGNATURES = {
     "hfee_post_norm": [P, P, F, P, F, F, P, F, P, I, P, P, P, I, I, P],
     "hfee_token_shift": [P, I, P, P, P, P, P, P, P, I, I, P],
     "hfee_softcap": [P, F, L, P],
+    "hfee_delta_inputs_fit": [I, I, I],
+    "hfee_delta_inputs": [P, L, P, P, P, L, P, P, I, P, P, I, P, P, P, P, P, I, I, I, I, I, F, F, I, P],
+    "hfee_delta_chunks": [P, L, P, P, L, P, L, P, L, P, L, P, L, P, P, P, I, I, I, I, I, I, I, I, P, L, P],
+    "hfee_delta_chunks_least": [],
     "hfee_group_norm": [P, I, P, P, P, F, I, I, I, P],
     "hfee_pair_norm_add": [P, P, P, P, P, F, F, F, P, I, P, F, I, I, I, P],
     "hfee_experts_join": [P, P, I, P, P, I, I, P, L, P, P, L, P, I, P, F, I, I, I, P],

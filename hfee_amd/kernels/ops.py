@@ -1653,6 +1653,48 @@ def linear_chunks_scratch(longest: int, rows: int, heads: int, dim: int) -> int:
     return heads * rows * LINEAR_CHUNK
 
 
+def delta_chunks_scratch(longest: int, rows: int, heads: int, dim: int, vdim: int) -> int:
+    """float32 words with which `linear_scan` walks the long portions of a step (the longest of `longest` tokens, `rows`
+    in all) of the delta rule with one decay a head in chunks; 0 where it has none."""
+    if not linear_chunks_fit(dim) or longest < int(lib.core().raw("hfee_delta_chunks_least")()):
+        return 0
+    return heads * rows * (LINEAR_CHUNK + dim + vdim + 2)
+
+
+def delta_inputs_fit(channels: int, dim: int, taps: int) -> bool:
+    """Whether `delta_inputs` takes these sizes (else: the short convolution, `unit_heads` and `scan_gate`)."""
+    return bool(lib.core().raw("hfee_delta_inputs_fit")(int(channels), int(dim), int(taps)))
+
+
+def delta_inputs(y, decay, beta, x, a, b, state, taps, dt_bias, a_log, token_segment, segment_rows, segment_slots,
+                 qk_width: int, dim: int, heads: int, unit_eps: float, q_factor: float, keep: bool):
+    """Everything that enters the gated delta rule with one decay a head, from the projections x ([n, channels]: queries,
+    keys, values), a and b ([n, heads], blocks of columns of x's buffer): y (float32 [n, channels]) =
+    `short_conv_silu` of x, queries and keys then unit vectors over each head of dim (eps unit_eps), queries times
+    q_factor; decay (float32 [n, heads]) = exp(-exp(a_log) * softplus(a + dt_bias)); beta = sigmoid(b).  keep: every row is its
+    segment's only token, and the state gets its input as by `short_conv_keep`."""
+    _gpu(y, decay, beta, x, a, b, state, taps, dt_bias, a_log, token_segment, segment_rows, segment_slots)
+    n, C, ldx = _rows2d(x, "delta_inputs x")
+    ny, wy, ldy = _f32rows(y, "delta_inputs y")
+    K = taps.shape[1]
+    _check(ny == n and wy == C and tuple(taps.shape) == (C, K) and taps.dtype == torch.float32 and taps.is_contiguous(), "delta_inputs: y and taps")
+    _check(state.dtype == x.dtype and state.is_contiguous() and tuple(state.shape[1:]) == (K - 1, C), "delta_inputs: state [slots, K - 1, C]")
+    for t in (decay, beta):
+        _check(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (n, heads), "delta_inputs: decay and beta float32 [n, heads]")
+    for t in (a, b):
+        na, wa, lda = _rows2d(t, "delta_inputs a, b")
+        _check(na == n and wa == heads and t.dtype == x.dtype and (n == 1 or lda == ldx), "delta_inputs: a and b are columns of x's buffer")
+    for t in (dt_bias, a_log):
+        _check(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == heads, "delta_inputs: dt_bias and a_log float32 [heads]")
+    _i32(token_segment, "delta_inputs token_segment", n)
+    _i32(segment_rows, "delta_inputs segment_rows")
+    _i32(segment_slots, "delta_inputs segment_slots")
+    _check(not keep or segment_rows.numel() == n, "delta_inputs: keep is for steps of single tokens")
+    lib.core().call("hfee_delta_inputs", _ptr(y), ldy, _ptr(decay), _ptr(beta), _ptr(x), ldx, _ptr(a), _ptr(b), _dt(x), _ptr(state),
+                    _ptr(taps), K, _ptr(dt_bias), _ptr(a_log), _ptr(token_segment), _ptr(segment_rows), _ptr(segment_slots), n, C,
+                    int(qk_width), int(dim), int(heads), float(unit_eps), float(q_factor), int(keep), _stream())
+
+
 def linear_scan(out, state, q, k, v, decay, beta, segment_rows, segment_lengths, segment_slots, heads: int,
                 qk_heads: int, dim: int, vdim: int, rule: str, decay_per_head: bool = False, longest: int = 0,
                 shortest: int = 0, scratch=None):
@@ -1664,7 +1706,7 @@ def linear_scan(out, state, q, k, v, decay, beta, segment_rows, segment_lengths,
     of a head's rows (or [heads]: the same decays for every token); beta [n, heads].
     With rule "decay_add" and the same decays for every token, `scratch` (float32, `linear_chunks_scratch` words) and
     the lengths of the step's longest and shortest portion: long portions go in chunks through the matrix cores,
-    in float32 as well."""
+    in float32 as well; likewise with rule "delta" and one decay a head and token (`delta_chunks_scratch` words)."""
     _gpu(out, state, q, k, v, decay, beta, segment_rows, segment_lengths, segment_slots)
     n, wq, ldq = _f32rows(q, "linear_scan q")
     nk, wk, ldk = _f32rows(k, "linear_scan k")
@@ -1692,9 +1734,19 @@ def linear_scan(out, state, q, k, v, decay, beta, segment_rows, segment_lengths,
     skip_from = 0
     if scratch is not None:
         _gpu(scratch)
-        _check(rule == "decay_add" and decay.dim() == 1, "linear_scan: only fixed decays go in chunks")
+        chunked_delta = rule == "delta" and decay_per_head and decay.dim() == 2
+        _check(chunked_delta or (rule == "decay_add" and decay.dim() == 1), "linear_scan: only fixed decays, and the delta rule with "
+               "one decay a head, go in chunks")
         _check(scratch.dtype == torch.float32 and scratch.is_contiguous() and 0 < shortest <= longest <= n, "linear_scan: scratch and lengths")
-        if ldq % 4 == 0 and ldk % 4 == 0 and q.data_ptr() % 16 == 0 and k.data_ptr() % 16 == 0:
+        aligned = ldq % 4 == 0 and ldk % 4 == 0 and q.data_ptr() % 16 == 0 and k.data_ptr() % 16 == 0
+        if aligned and chunked_delta:
+            skip_from = int(lib.core().raw("hfee_delta_chunks_least")())
+            lib.core().call("hfee_delta_chunks", _ptr(out), ldo, _ptr(state), _ptr(q), ldq, _ptr(k), ldk, _ptr(v), ldv, _ptr(decay), ldd,
+                            _ptr(beta), ldb, _ptr(segment_rows), _ptr(segment_lengths), _ptr(segment_slots), segments, int(longest), n,
+                            heads, qk_heads, dim, vdim, _scan_rows_a_lane(dim), _ptr(scratch), scratch.numel(), _stream())
+            if shortest >= skip_from:
+                return
+        elif aligned:
             skip_from = int(lib.core().raw("hfee_linear_chunks_least")())
             lib.core().call("hfee_linear_chunks", _ptr(out), ldo, _ptr(state), _ptr(q), ldq, _ptr(k), ldk, _ptr(v), ldv, _ptr(decay),
                             _ptr(segment_rows), _ptr(segment_lengths), _ptr(segment_slots), segments, int(longest), n, heads,

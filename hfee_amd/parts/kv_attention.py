@@ -295,7 +295,7 @@ class KvAttention(_KvMixer):
         else:       # this run of the layer reads keys and values that another run wrote
             ops.linear(q, hn, self.w_qkv[:self.q_width])
             k = v = None
-        if self.prepares:
+        if self.prepares or (self.blend is None and self.pairing):
             made = ctx.rows("kv_attention.q", self.q_width)
             ops.qkv_write(made, q, k, v, ctx.positions, ctx.token_segment, tables, cos, sin, cache, H, G, dk, dv, ctx.page_size,
                           ctx.max_position, biases=self.biases, norm=self.qk_norm, q_weight=self.q_norm, k_weight=self.k_norm,

@@ -151,6 +151,9 @@ class GatedDelta(_StateMixer):
         self.a_columns = slice(self.channels, second) if self.gate_rank is not None else slice(second, self.at_b)
         self.g_columns = slice(second, self.at_b) if self.gate_rank is not None else slice(self.channels, second)
         self.conv_taps = torch.cat([f32(n["q_conv"]), f32(n["k_conv"]), f32(n["v_conv"])], dim=0).contiguous()
+        # (what enters the recurrence is one launch where its kernel takes the sizes)
+        self.one_launch = (self.decay_per_head and self.w_in.is_cuda and self.w_in.shape[0] % 8 == 0
+                           and ops.delta_inputs_fit(self.channels, self.dim, self.taps))
         self.a_log, self.dt_bias, self.norm_weight = f32(n["a_log"]), f32(n["dt_bias"]), f32(n["norm"])
         self.w_o = tensors.pop(n["o"]).contiguous()
         self.w_in_tiles, = tiles_of(self.dtype, self.w_in)
@@ -183,24 +186,23 @@ class GatedDelta(_StateMixer):
         proj = ctx.rows("gated_delta.in", self.w_in.shape[0])
         product(ctx, proj, hn, self.w_in, self.w_in_tiles)
         raw = proj[:, :self.channels]
-        y = ctx.rows("gated_delta.conv", self.channels, torch.float32)
-        ops.short_conv_silu(y, raw, self.conv_state, self.conv_taps, ctx.token_segment, rows, slots)
-        ops.short_conv_keep(self.conv_state, raw, rows, lengths, slots)
-        q, k, v = y[:, :self.qk_width], y[:, self.qk_width:2 * self.qk_width], y[:, 2 * self.qk_width:]
-        ops.unit_heads(q, G, D, self.unit_eps, D ** -0.5)
-        ops.unit_heads(k, G, D, self.unit_eps, 1.0)
-        per_decay = 1 if self.decay_per_head else D
-        step = proj[:, self.a_columns]
-        if not self.decay_per_head:
-            step = ctx.rows("gated_delta.step", H * D)
-            product(ctx, step, proj[:, self.a_columns], self.w_a_up, self.w_a_up_tiles)
-        decay = ctx.rows("gated_delta.decay", H * per_decay, torch.float32)
-        ops.scan_gate(decay, step, "step_decay", bias=self.dt_bias, per_head=self.a_log, head_width=per_decay)
+        # (rows that the recurrence's kernels for long portions read in columns)
+        y = ctx.rows("gated_delta.conv", staggered(self.channels), torch.float32)[:, :self.channels]
         beta = ctx.rows("gated_delta.beta", H, torch.float32)
-        ops.scan_gate(beta, proj[:, self.at_b:self.at_b + H], "sigmoid")
-        o = ctx.rows("gated_delta.read", self.v_width, torch.float32)
+        if self.one_launch:
+            decay = ctx.rows("gated_delta.decay", H, torch.float32)
+            singles = ctx.n == len(ctx.segments)
+            ops.delta_inputs(y, decay, beta, raw, proj[:, self.a_columns], proj[:, self.at_b:self.at_b + H], self.conv_state,
+                             self.conv_taps, self.dt_bias, self.a_log, ctx.token_segment, rows, slots, self.qk_width, D, H,
+                             self.unit_eps, D ** -0.5, keep=singles)
+            if not singles:
+                ops.short_conv_keep(self.conv_state, raw, rows, lengths, slots)
+        else:
+            decay = self._inputs(ctx, y, beta, proj)
+        q, k, v = y[:, :self.qk_width], y[:, self.qk_width:2 * self.qk_width], y[:, 2 * self.qk_width:]
+        o = ctx.rows("gated_delta.read", staggered(self.v_width), torch.float32)[:, :self.v_width]
         ops.linear_scan(o, self.state, q, k, v, decay, beta, rows, lengths, slots, H, G, D, V, "delta",
-                        decay_per_head=self.decay_per_head)
+                        decay_per_head=self.decay_per_head, **self._delta_chunks(ctx))
         gate = proj[:, self.g_columns]
         if self.gate_rank is not None:
             gate = ctx.rows("gated_delta.gate", self.v_width)
@@ -208,6 +210,35 @@ class GatedDelta(_StateMixer):
         gated = ctx.rows("gated_delta.out", self.v_width)
         ops.head_norm_gate(gated, o, gate, self.norm_weight, H, V, self.norm_eps, self.gate_activation)
         product(ctx, x, gated, self.w_o, self.w_o_tiles, add=add)
+
+    def _delta_chunks(self, ctx) -> dict:
+        """The arguments with which `ops.linear_scan` walks a step's long portions in chunks (one decay a head only)."""
+        if not self.decay_per_head:
+            return {}
+        lengths = [s.length for s in ctx.segments]
+        words = ops.delta_chunks_scratch(max(lengths), ctx.n, self.heads, self.dim, self.vdim)
+        if not words:
+            return {}
+        return dict(scratch=ctx.workspace.flat("recurrent.chunks", words, torch.float32), longest=max(lengths), shortest=min(lengths))
+
+    def _inputs(self, ctx, y, beta, proj):
+        """What enters the recurrence, a launch a mechanism: fills y and beta, returns the decays."""
+        H, G, D = self.heads, self.qk_heads, self.dim
+        rows, lengths, slots = self._segments(ctx)
+        raw = proj[:, :self.channels]
+        ops.short_conv_silu(y, raw, self.conv_state, self.conv_taps, ctx.token_segment, rows, slots)
+        ops.short_conv_keep(self.conv_state, raw, rows, lengths, slots)
+        ops.unit_heads(y[:, :self.qk_width], G, D, self.unit_eps, D ** -0.5)
+        ops.unit_heads(y[:, self.qk_width:2 * self.qk_width], G, D, self.unit_eps, 1.0)
+        per_decay = 1 if self.decay_per_head else D
+        step = proj[:, self.a_columns]
+        if not self.decay_per_head:
+            step = ctx.rows("gated_delta.step", H * D)
+            product(ctx, step, proj[:, self.a_columns], self.w_a_up, self.w_a_up_tiles)
+        decay = ctx.rows("gated_delta.decay", H * per_decay, torch.float32)
+        ops.scan_gate(decay, step, "step_decay", bias=self.dt_bias, per_head=self.a_log, head_width=per_decay)
+        ops.scan_gate(beta, proj[:, self.at_b:self.at_b + H], "sigmoid")
+        return decay
 
 
 @register_mixer("gla")
