@@ -1290,10 +1290,10 @@ def pair_norm_add(x, y, y2, weight, weight2, eps: float, scales=(1.0, 1.0), next
                     float(eps), *_next_norm(next_out, next_weight, next_eps, next_groups, n, d, "pair_norm_add"), n, d, _stream())
 
 
-def experts_join(x, y, chosen, weights, experts: int, h, shared=None, gate=None, next_out=None, next_weight=None,
-                 next_eps: float = 0.0, next_groups: int = 1):
+def experts_join(x, y, chosen, weights, experts: int, h, summed: bool = False, shared=None, gate=None, next_out=None,
+                 next_weight=None, next_eps: float = 0.0, next_groups: int = 1):
     """x[t] (float32, the residual stream) += what a token's experts make of it.  y: float32 [n * top, d], the outputs
-    of the (token, expert) pairs, or [n, d], their weighted sum; chosen int32 [n, top], weights float32 [n, top]:
+    of the (token, expert) pairs, or with `summed` [n, d], their weighted sum; chosen int32 [n, top], weights float32 [n, top]:
     numbers at and beyond `experts` are experts without matrices that hand on their input h [n, d] (times the
     weight; their rows of y are not looked at).  shared: float32 [n, d], added too, with gate (float32, one number a
     row, any stride) times sigmoid(gate[t]).  next_out, ...: as in `pair_norm_add`; next_out and h share a dtype."""
@@ -1302,9 +1302,8 @@ def experts_join(x, y, chosen, weights, experts: int, h, shared=None, gate=None,
     nh, wh, ldh = _rows2d(h, "experts_join h")
     top = chosen.shape[1]
     _check(x.dtype == torch.float32 and x.is_contiguous() and nh == n and wh == d, "experts_join: contiguous float32 x, h of its shape")
-    _check(y.dtype == torch.float32 and y.is_contiguous() and y.dim() == 2 and y.shape[1] == d and y.shape[0] in (n, n * top),
-           "experts_join: y float32 [n * top, d] or [n, d]")
-    summed = y.shape[0] == n and top > 1
+    _check(y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (n if summed else n * top, d),
+           "experts_join: y float32 [n * top, d], or summed [n, d]")
     _check(chosen.dtype == torch.int32 and chosen.is_contiguous() and tuple(chosen.shape) == (n, top), "experts_join: chosen int32 [n, top]")
     _check(weights.dtype == torch.float32 and weights.is_contiguous() and tuple(weights.shape) == (n, top), "experts_join: weights float32 [n, top]")
     if shared is not None:

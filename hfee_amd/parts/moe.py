@@ -228,7 +228,8 @@ class RoutedMoE(FeedForward):
             shared = ctx.rows("routed_moe.shared", self.hidden, torch.float32)
             self.shared.forward_into(ctx, shared, hn)
         chosen, weights, gate = self._choose(ctx, hn)
-        if self._grouped(n, hn):
+        grouped = self._grouped(n, hn)
+        if grouped:
             order = ws.flat("table_moe.order", ws.capacity * top, torch.int32)
             tiles = ws.flat("table_moe.tiles", 3 * ops.moe_group_tiles(ws.capacity, top, self.experts) + 1, torch.int32)
             act = ctx.rows("table_moe.act", top * self.intermediate)
@@ -239,7 +240,7 @@ class RoutedMoE(FeedForward):
             ops.moe_up(act, hn, self.w_gate, self.w_up, top, chosen=chosen, **self.gate)
             y = ctx.rows("routed_moe.summed", self.hidden, torch.float32)
             ops.moe_down(y, act, self.w_down, top, pair_weights=weights, chosen=chosen, accumulate=False)
-        ops.experts_join(x, y, chosen, weights, self.experts, hn, shared=shared, gate=gate,
+        ops.experts_join(x, y, chosen, weights, self.experts, hn, summed=not grouped, shared=shared, gate=gate,
                          **(then.offer_rows() if then is not None else {}))
 
     def _run(self, ctx, out, h, add: bool):

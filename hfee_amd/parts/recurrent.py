@@ -121,17 +121,17 @@ class GatedDelta(_StateMixer):
                  TensorSpec(n["k"], (self.qk_width, self.hidden)), TensorSpec(n["k_conv"], (self.qk_width, self.taps), role="vector"),
                  TensorSpec(n["v"], (self.v_width, self.hidden)), TensorSpec(n["v_conv"], (self.v_width, self.taps), role="vector"),
                  TensorSpec(n["b"], (H, self.hidden)), TensorSpec(n["a_log"], (H,), role="vector"),
-                 TensorSpec(n["norm"], (self.vdim,), role="vector", init=("one_plus_normal",)),
-                 TensorSpec(n["dt_bias"], (H if self.decay_per_head else H * D,), role="vector"),
-                 TensorSpec(n["o"], (self.hidden, self.v_width))]
+                 TensorSpec(n["norm"], (self.vdim,), role="vector", init=("one_plus_normal",))]
         if self.decay_per_head:
             specs.append(TensorSpec(n["a"], (H, self.hidden)))
         else:
             specs += [TensorSpec(n["a_down"], (self.decay_rank, self.hidden)), TensorSpec(n["a_up"], (H * D, self.decay_rank))]
+        specs.append(TensorSpec(n["dt_bias"], (H if self.decay_per_head else H * D,), role="vector"))
         if self.gate_rank is None:
             specs.append(TensorSpec(n["g"], (self.v_width, self.hidden)))
         else:
             specs += [TensorSpec(n["g_down"], (self.gate_rank, self.hidden)), TensorSpec(n["g_up"], (self.v_width, self.gate_rank))]
+        specs.append(TensorSpec(n["o"], (self.hidden, self.v_width)))
         return specs
 
     def bind(self, tensors):
@@ -152,18 +152,18 @@ class GatedDelta(_StateMixer):
         self.g_columns = slice(second, self.at_b) if self.gate_rank is not None else slice(self.channels, second)
         self.conv_taps = torch.cat([f32(n["q_conv"]), f32(n["k_conv"]), f32(n["v_conv"])], dim=0).contiguous()
         # (what enters the recurrence is one launch where its kernel takes the sizes)
-        self.one_launch = (self.decay_per_head and self.w_in.is_cuda and self.w_in.shape[0] % 8 == 0
+        self.one_launch = (self.decay_per_head and self.w_in.is_cuda
                            and ops.delta_inputs_fit(self.channels, self.dim, self.taps))
         self.a_log, self.dt_bias, self.norm_weight = f32(n["a_log"]), f32(n["dt_bias"]), f32(n["norm"])
         self.w_o = tensors.pop(n["o"]).contiguous()
-        self.w_in_tiles, = tiles_of(self.dtype, self.w_in)
-        self.w_o_tiles, = tiles_of(self.dtype, self.w_o)
+        self.w_in_tiles, self.w_o_tiles = tiles_of(self.dtype, self.w_in, self.w_o)
+        halves = [n[r] for r, has in (("a_up", not self.decay_per_head), ("g_up", self.gate_rank is not None)) if has]
+        ups = [tensors.pop(name).contiguous() for name in halves]
+        tiles = list(tiles_of(self.dtype, *ups)) if ups else []
         if not self.decay_per_head:
-            self.w_a_up = tensors.pop(n["a_up"]).contiguous()
-            self.w_a_up_tiles, = tiles_of(self.dtype, self.w_a_up)
+            self.w_a_up, self.w_a_up_tiles = ups.pop(0), tiles.pop(0)
         if self.gate_rank is not None:
-            self.w_g_up = tensors.pop(n["g_up"]).contiguous()
-            self.w_g_up_tiles, = tiles_of(self.dtype, self.w_g_up)
+            self.w_g_up, self.w_g_up_tiles = ups.pop(0), tiles.pop(0)
 
     def state_specs(self):
         return [(self.prefix + "state", (self.heads, *ops.scan_state_shape(self.dim, self.vdim)), torch.float32),
