@@ -204,7 +204,7 @@ __global__ __launch_bounds__(kScanWaves * 64) void linear_scan_kernel(
   typedef ScanShape<DPT> Sh;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int seg = blockIdx.z, h = blockIdx.y, tid = threadIdx.x;
-  if (skip_from > 0 && segment_lengths[seg] >= skip_from) return;       // (linear_chunks.hip has this portion)
+  if (skip_from > 0 && segment_lengths[seg] >= skip_from) return;       // (linear_chunks.hip or delta_chunks.hip has this portion)
   const int lane = tid & 63, wave = tid >> 6;
   const int part = lane & (kScanParts - 1), c = lane >> 4;
   const int block = blockIdx.x * kScanWaves + wave;                 // of four columns
